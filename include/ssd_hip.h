@@ -31,7 +31,7 @@ extern "C" {
 
 /* Bumped whenever a signature or a semantic of this header changes; ssd_abi_version() returns the value the library was built
  * with, so a consumer compiled against another header can tell (tests/abi_consumer.c does). */
-#define SSD_HIP_ABI_VERSION 6
+#define SSD_HIP_ABI_VERSION 7
 
 #define SSD_OK 0
 #define SSD_ERR_SHAPE (-1)
@@ -431,6 +431,10 @@ int ssd_moe_combine(const void* y_rows, const int32_t* inv, const float* weights
  * stride ldx) by w_rows + g * N * K and writes y + g * gsy (row stride ldy; strides in elements of the respective type). */
 int ssd_gemm_rows_batched(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, int G, long ldx, long gsx, long ldy,
                           long gsy, int epilogue, int f32, void* stream);
+/* One product whose columns feed a recurrence: y fp32 [M][N], columns n < n_decay = exp(-rate[n] * softplus(z + bias[n])), the others
+ * 1 / (1 + exp(-z)), z = <x_row, w_row n>; rate and bias fp32 [n_decay]. */
+int ssd_gemm_rows_decay_gate(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, const float* rate, const float* bias,
+                             int n_decay, int f32, void* stream);
 
 /* Parallel layers with Dynamic-Tanh norms, dyt(x) = tanh(alpha * x) * weight + bias (csrc/dyt.hip); alpha: one fp32 number in
  * device memory.  ssd_dyt_embed: x (fp32 [T][W]) = dyt(table[ids]); x0 (optional) a second fp32 copy; cat (optional) an element-type
@@ -447,8 +451,8 @@ int ssd_parallel_tail(void* x, const void* y_mix, const void* y_ff, const void* 
                       int top, const void* shared_rows, const float* shared_gate, long ld_shared_gate, const float* next_alpha,
                       const void* next_weight, const void* next_bias, void* next_out, void* cat, long ld_cat, int T, int W, int f32,
                       void* stream);
-/* out[r][c] = act(ab[r][c]) * ab[r][F + c] for fp32 rows [rows][2F]; act 0: silu, 1: tanh-form gelu. */
-int ssd_glu_rows(const void* ab_rows, void* out_rows, int rows, int F, int act, int f32, void* stream);
+/* out[r * ldo + c] = act(ab[r][c]) * ab[r][F + c] for fp32 rows [rows][2F]; act 0: silu, 1: tanh-form gelu. */
+int ssd_glu_rows(const void* ab_rows, void* out_rows, long ldo, int rows, int F, int act, int f32, void* stream);
 
 /* Latent attention with a sliding window (csrc/attention_latent.hip).  proj_rows fp32 [T][ld] = [dq (q_rank) | latent (kv_rank) |
  * rotated key part (rot) | gate logits (H)].  Store: cq_out [T][q_rank] = rms(dq) * q_norm_w; cache row slots[t] (-1: none) of
@@ -529,15 +533,18 @@ int ssd_moe_route_sigmoid_grouped(const float* logits, long ld, const float* cor
  * K cache [blocks][G][block_size][D] row slots[t] (-1: none) = k / rms(k); V cache [blocks][G][Dv][block_size] (transposed per page).
  * Attention: out[t][h] (Dv wide) = sum_j p_j v_j over the keys j of the token's sequence with 0 <= positions[t] - j < window
  * (window 0: all keys up to the token), s_j = cap * tanh(scale * <q, k_j> / cap) - slopes[h] * (positions[t] - j) (cap <= 0: no cap;
- * slopes NULL: no penalty), p_j = exp(s_j) / (sum_j' exp(s_j') + exp(sinks[h])) (sinks NULL: no sink).  max_q > 0 (an upper bound of
+ * slopes NULL: no penalty), p_j = exp(s_j) / (sum_j' exp(s_j') + exp(sinks[h])) (sinks NULL: no sink).  keep_first > 0: keys j <
+ * keep_first stay visible whatever the window.  gate_rows (fp32, row stride ldg, NULL: none): the output entries are multiplied by
+ * sigmoid(gate_rows[t * ldg + h * Dv + d]) * out_scale.  Output rows have row stride ldo.  max_q > 0 (an upper bound of
  * the rows any sequence of the batch brings) admits the MFMA form for bf16 and D % 32 == 0, Dv % 16 == 0, block_size % 32 == 0; max_q = 0
  * or other sizes or fp32: the scalar form. */
 int ssd_winattn_store(const void* qkv_rows, long ld, float eps, const int32_t* slots, void* q_out, void* k_cache, void* v_cache, int T,
                       int H, int G, int D, int Dv, int block_size, int f32, void* stream);
 int ssd_winattn_paged(const void* q_rows, const void* k_cache, const void* v_cache, const float* slopes, const float* sinks,
                       const int32_t* block_tables, int max_blocks, const int64_t* positions, const int32_t* cu_q, int q_per_seq,
-                      int max_q, int B, int T, int H, int G, int D, int Dv, int block_size, int window, float scale, float cap,
-                      const float* out_freqs, void* out_rows, int f32, void* stream);
+                      int max_q, int B, int T, int H, int G, int D, int Dv, int block_size, int window, int keep_first, float scale,
+                      float cap, const float* out_freqs, const float* gate_rows, long ldg, float out_scale, void* out_rows, long ldo,
+                      int f32, void* stream);
 /* The store of the rotary variant: q_out = rope(q_norm_w * q / rms(q)) with the RMS over ALL H * D entries of the row's q (k alike,
  * over G * D, into the K cache); rope turns the first rot_dims entries of every head (entry i pairs with i + rot_dims / 2) by
  * positions[t] * qk_freqs[i].  v_freqs (fp32 [Dv / 2], NULL: none): every value head turns over all Dv entries by positions[t] *
@@ -546,6 +553,13 @@ int ssd_winattn_paged(const void* q_rows, const void* k_cache, const void* v_cac
 int ssd_winattn_store_rope(const void* qkv_rows, long ld, const void* q_norm_w, const void* k_norm_w, float eps, const int64_t* positions,
                            const float* qk_freqs, int rot_dims, const float* v_freqs, const int32_t* slots, void* q_out, void* k_cache,
                            void* v_cache, int T, int H, int G, int D, int Dv, int block_size, int f32, void* stream);
+/* The store of a variant with short causal convolutions and no norms: every channel of q, k and v (columns col_off .. of proj_rows fp32
+ * [T][ld] in that order; channels 0 .. of conv_w [C][taps] and of conv_state fp32 [slots][taps - 1][C]) becomes sum_j conv_w[c][j] *
+ * in[t - (taps - 1 - j)][c]; then the first rot_dims entries of every q / k head turn.  conv_state is only read. */
+int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int col_off, const void* conv_w, int taps, const float* conv_state, int C,
+                                const int32_t* state_slots, const int64_t* positions, const int32_t* cu_q, int q_per_seq, int B,
+                                const float* qk_freqs, int rot_dims, const int32_t* slots, void* q_out, void* k_cache, void* v_cache,
+                                int T, int H, int G, int D, int Dv, int block_size, int f32, void* stream);
 
 /* Layers that normalise a sublayer's output only, with a weighted average over the depth (csrc/postnorm.hip).
  * ssd_embed_hist: x_out fp32 [T][W] = table[ids[t]] (zeros for an id outside the table), the same into hist0 (optional) and as
@@ -582,8 +596,9 @@ int ssd_gate_rows(const void* o_rows, long ldo, const void* gate_rows, long ldg,
  * dt B x^T over state fp32 [slots][H][N][Dv], y = S^T C + skip[h] x; x / B / C = xbc_rows fp32 [T][ldx] at x_off ([H][Dv]), b_off,
  * c_off ([G][N] each); out fp32 [T][H*Dv]; also saves the last taps - 1 rows of proj_rows columns conv_off .. conv_off + C into
  * conv_state[slot].
- * ssd_group_gate_norm: rows of N entries in `groups` equal parts, g = silu(gate_rows[t][c]) (fp32, row stride ldg): gate_first ?
- * weight * rms_part(o * g) : weight * rms_part(o) * g, element-type rows. */
+ * ssd_group_gate_norm: rows of N entries in `groups` equal parts, g = act(gate_rows[t][c]) (fp32, row stride ldg; gate_act 0: silu, 1:
+ * sigmoid, 2: the entry itself): out_scale * (gate_first ? weight * rms_part(o * g) : weight * rms_part(o) * g), element-type rows of
+ * stride ldo; w_period > 0: weight holds w_period entries, repeated along the row. */
 int ssd_token_shift_mix(const void* hn_rows, const void* mu, const float* shift_state, const int64_t* positions, const int32_t* cu_q,
                         int q_per_seq, const int32_t* state_slots, int B, void* out_rows, int T, int W, int S, int f32, void* stream);
 int ssd_wkv_scan(const void* proj_rows, long ld, int r_off, int k_off, int v_off, const void* decay_rows, long ldw, const float* w0,
@@ -596,8 +611,40 @@ int ssd_ssd_scan(const void* xbc_rows, long ldx, int x_off, int b_off, int c_off
                  const float* dt_bias, const float* a_log, const float* skip, const int64_t* positions, const int32_t* cu_q,
                  int q_per_seq, const int32_t* state_slots, void* state, void* out_rows, int conv_off, int C, void* conv_state,
                  int taps, int B, int H, int G, int N, int Dv, void* stream);
-int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, const void* weight, float eps, void* out_rows, int T,
-                        int N, int groups, int gate_first, int f32, void* stream);
+int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, int gate_act, const void* weight, int w_period, float eps,
+                        float out_scale, void* out_rows, long ldo, int T, int N, int groups, int gate_first, int f32, void* stream);
+
+/* Gated delta rule over per-sequence state slots (csrc/delta.hip): per head h (q / k head h / (H / G)) over a state of D key channels x
+ * Dv value columns, S <- decay S (decay: one number per head, or one per key channel), u = beta (v - S^T k), S <- S + k u^T,
+ * o = S^T q.  Heads' key channels are padded with zeros to DP = 32 (D <= 32) or the next multiple of 64 (D <= 512).
+ * ssd_delta_prep: from proj_rows fp32 [T][ld]: columns col_off .. = q (G*D) | k (G*D) | v (H*Dv), each channel through silu(sum_j
+ * conv_w[c][j] * in[t - (taps - 1 - j)][c]) (conv_w [2GD + HDv][taps]; inputs before a portion from channels conv_c0 .. of conv_state
+ * fp32 [slots][taps - 1][C], only read); q and k divided by sqrt(sum of squares + 1e-6) per head, q also by sqrt(D).  qk_rows fp32
+ * [T][G][2][DP] (q, then k), v_rows fp32 [T][H*Dv], scalars fp32 [T][H][4] = {sigmoid(proj[b_off + h]), exp(-rate[h] *
+ * softplus(proj[a_off + h] + bias[h])) (a_off < 0: 1), <q, k>, 0}; lr_out (optional): element-type rows [T][ld_lr] = proj columns
+ * lr_off .. lr_off + lr_n, then zeros.
+ * ssd_delta_scan: state fp32 [slots][H][Dv][DP]; decay_rows fp32 [T][ldd] with the per-channel decays of head h at h * DP (NULL: the
+ * scalars' decay); out fp32 [T][H*Dv]; also saves the last taps - 1 rows of proj_rows columns conv_off .. conv_off + C into
+ * conv_state[slot]. */
+int ssd_delta_prep(const void* proj_rows, long ld, int col_off, const void* conv_w, int taps, const float* conv_state, int C, int conv_c0,
+                   const int32_t* state_slots, const int64_t* positions, const int32_t* cu_q, int q_per_seq, int B, int b_off, int a_off,
+                   const float* rate, const float* bias, int lr_off, int lr_n, void* lr_out, long ld_lr, void* qk_rows, void* v_rows,
+                   void* scalars, int T, int H, int G, int D, int Dv, int DP, int f32, void* stream);
+int ssd_delta_scan(const void* qk_rows, const void* v_rows, const void* scalars, const float* decay_rows, long ldd,
+                   const int64_t* positions, const int32_t* cu_q, int q_per_seq, const int32_t* state_slots, void* state, void* out_rows,
+                   int B, int H, int G, int D, int Dv, int DP, const void* proj_rows, long ld, int conv_off, int C, void* conv_state,
+                   int taps, void* stream);
+
+/* Layer norm over an fp32 residual with one or two weight sets per statistic (csrc/layernorm.hip): out = (x - mean) / sqrt(var + eps) *
+ * w + b as element-type rows; out1 / out2 may be NULL (out2 only with out1).
+ * ssd_lnorm_embed: x_out fp32 [T][W] = table[ids[t]] (zeros for an id outside the table) first; ssd_lnorm_tail: x += mult * y_rows
+ * (fp32) first; ssd_lnorm_rows: out_rows[r] = the norm of x[gather[r]] (or x[r]). */
+int ssd_lnorm_embed(const int64_t* ids, const void* table, void* x_out, const void* w1, const void* b1, void* out1, const void* w2,
+                    const void* b2, void* out2, float eps, int T, int W, long vocab, int f32, void* stream);
+int ssd_lnorm_tail(void* x, const void* y_rows, float mult, const void* w1, const void* b1, void* out1, const void* w2, const void* b2,
+                   void* out2, float eps, int T, int W, int f32, void* stream);
+int ssd_lnorm_rows(const void* x, const void* weight, const void* bias, void* out_rows, const int32_t* gather, float eps, int T, int W,
+                   int f32, void* stream);
 
 /* hipGraph capture for a host that is not PyTorch -- the reference captures its decode / verify / glue / tree steps with
  * torch.cuda.CUDAGraph (ssd/engine/helpers/cudagraph_helpers.py:20-120); every entry point above only enqueues on `stream`, so the calls

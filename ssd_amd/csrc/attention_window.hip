@@ -18,9 +18,15 @@
 //                         every value head turned by its own position over all Dv entries before it is cached; the attention then
 //                         turns every head's output back by the query's position (out_freqs), so that the weighted sum carries
 //                         relative positions.  Pairs are (i, i + n / 2) throughout.
+//   * ssd_winattn_store_conv_rope  the store of a variant without norms: a short causal convolution over time on every channel of q, k and
+//                         v (the inputs of earlier tokens from the sequence's slot), then rotary positions on q and k.
+//   keep_first > 0: the sequence's first keep_first tokens stay visible whatever the window (they keep their true positions); the walk
+//   then starts with those of them that lie before the window.  gate (fp32 rows, one entry per output entry): the heads' outputs are
+//   multiplied by sigmoid(gate) * out_scale; the output rows have a row stride.
 //   Scores, weights, sums and norms are fp32 whatever the element type.  A token's position and sequence come from positions[] and
 //   cu_q[] (varlen batches: prompt portions beside single tokens) or q_per_seq (fixed rows per sequence).
 #include "common.h"
+#include "shortconv.h"
 
 namespace {
 
@@ -133,11 +139,53 @@ winattn_store_rope_kernel(const float* __restrict__ qkv, long ld, const T* __res
   }
 }
 
-__device__ __forceinline__ int seq_of_row(const int32_t* cu_q, int q_per_seq, int B, int t) {
-  if (!cu_q) return t / q_per_seq;
-  int lo = 0, hi = B;
-  while (hi - lo > 1) { const int mid = (lo + hi) >> 1; if (cu_q[mid] <= t) lo = mid; else hi = mid; }
-  return lo;
+// Short causal convolutions on every channel of q, k and v (csrc/shortconv.h; weights conv_w [C][taps] with the channels in the row's
+// order q | k | v), then the pair (i, i + half) of every q / k head turns by pos * qk_freqs[i].  The channels' columns start at col_off of
+// the projection rows; they are channels 0 .. of conv_state's C.  grid = (tokens, column blocks); the pairs' sines and cosines are
+// computed once per workgroup.
+template <typename T>
+__global__ void __launch_bounds__(256)
+winattn_store_conv_rope_kernel(const float* __restrict__ proj, long ld, int col_off, const T* __restrict__ cw, int taps,
+                               const float* __restrict__ conv_state, int C, const int32_t* __restrict__ state_slots,
+                               const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q, int q_per_seq, int B,
+                               const float* __restrict__ qk_freqs, int rot_dims, const int32_t* __restrict__ slots, T* __restrict__ q_out,
+                               T* __restrict__ kc, T* __restrict__ vc, int H, int G, int D, int Dv, int bs) {
+  __shared__ float sn[512], cs[512];
+  const int t = blockIdx.x;
+  const int b = seq_of_row(cu_q, q_per_seq, B, t);
+  const int row0 = cu_q ? cu_q[b] : b * q_per_seq;
+  const long p0 = positions[row0];
+  const float* st = conv_state + (size_t)state_slots[b] * (taps - 1) * C;
+  const float pos = (float)positions[t];
+  const int half = rot_dims >> 1;
+  for (int i = threadIdx.x; i < half; i += 256) sincosf(pos * qk_freqs[i], &sn[i], &cs[i]);
+  __syncthreads();
+  const int Nq = H * D, Nk = G * D;
+  const int slot = slots[t];
+  const long blk = slot >= 0 ? slot / bs : 0;
+  const int off = slot >= 0 ? slot % bs : 0;
+  const int per = D - half;                                // items of a q / k head: `half` pairs, then the entries that do not turn
+  const int n_qk = (H + G) * per, n_all = n_qk + (slot >= 0 ? G * Dv : 0);
+  auto val = [&](int c) { return conv_at<T>(proj, ld, (long)col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, 0.f); };
+  for (int u = blockIdx.y * 256 + threadIdx.x; u < n_all; u += 256 * gridDim.y) {
+    if (u < n_qk) {
+      const int hd = u / per, i = u % per;
+      const bool isq = hd < H;
+      if (!isq && slot < 0) continue;
+      const int base = hd * D;                             // k heads follow the q heads in the row
+      T* dst = isq ? q_out + (size_t)t * Nq + base : kc + (((size_t)blk * G + (hd - H)) * bs + off) * D;
+      if (i < half) {
+        const float a = val(base + i), b2 = val(base + i + half);
+        stf<T>(dst + i, a * cs[i] - b2 * sn[i]);
+        stf<T>(dst + i + half, b2 * cs[i] + a * sn[i]);
+      } else {
+        stf<T>(dst + i + half, val(base + i + half));
+      }
+    } else {
+      const int c = u - n_qk, g = c / Dv, d = c % Dv;
+      stf<T>(vc + (((size_t)blk * G + g) * Dv + d) * bs + off, val(Nq + Nk + c));
+    }
+  }
 }
 
 template <typename T>
@@ -145,7 +193,8 @@ __global__ void __launch_bounds__(256)
 winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc, const float* __restrict__ slopes,
                      const float* __restrict__ sinks, const int32_t* __restrict__ bt, int max_blocks,
                      const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q, int q_per_seq, int B, int H, int G, int D,
-                     int Dv, int bs, int window, float scale, float cap, const float* __restrict__ out_freqs, T* __restrict__ out) {
+                     int Dv, int bs, int window, int keep_first, float scale, float cap, const float* __restrict__ out_freqs,
+                     const float* __restrict__ gate, long ldg, float out_scale, T* __restrict__ out, long ldo) {
   extern __shared__ float smem[];
   const int t = blockIdx.x, h = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int g = h / (H / G);
@@ -158,7 +207,8 @@ winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T*
   const int b = seq_of_row(cu_q, q_per_seq, B, t);
   const int pos = (int)positions[t];
   const int first = window > 0 && pos + 1 > window ? pos + 1 - window : 0;
-  const int nkeys = pos + 1 - first;
+  const int nkept = min(keep_first, first);    // kept first tokens that the window no longer covers come before it in the walk
+  const int nkeys = nkept + pos + 1 - first;
   const int32_t* table = bt + (size_t)b * max_blocks;
   const float slope = slopes ? slopes[h] : 0.f;
 
@@ -174,7 +224,7 @@ winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T*
   long* rowp = srow + wave * 64;
   const int ntiles = (nkeys + 63) >> 6;
   for (int kt = wave; kt < ntiles; kt += 4) {
-    const int j = first + kt * 64 + lane;
+    const int ji = kt * 64 + lane, j = ji < nkept ? ji : first + ji - nkept;
     float s = -INFINITY;
     long crow = 0;
     if (j <= pos) {
@@ -238,7 +288,8 @@ winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T*
       sincosf((float)pos * out_freqs[d < hv ? d : d - hv], &sn, &c);
       s = d < hv ? s * c + o * sn : s * c - o * sn;
     }
-    stf<T>(out + ((size_t)t * H + h) * Dv + d, s);
+    if (gate) s = s / (1.0f + expf(-gate[(size_t)t * ldg + h * Dv + d])) * out_scale;
+    stf<T>(out + (size_t)t * ldo + h * Dv + d, s);
   }
 }
 
@@ -263,7 +314,8 @@ __global__ void __launch_bounds__(256)
 winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vt,
                     const float* __restrict__ slopes, const float* __restrict__ sinks, const int32_t* __restrict__ bt, int max_blocks,
                     const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q, int q_per_seq, int H, int G, int D, int Dv,
-                    int bs, int window, float scale, float cap, const float* __restrict__ out_freqs, bf16_t* __restrict__ out) {
+                    int bs, int window, int keep_first, float scale, float cap, const float* __restrict__ out_freqs,
+                    const float* __restrict__ gate, long ldg, float out_scale, bf16_t* __restrict__ out, long ldo) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, qd = lane >> 4;
   const int b = blockIdx.z, g = blockIdx.y, R = H / G;
@@ -300,8 +352,10 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
   const float inv_cap = cap > 0.f ? 1.0f / cap : 0.f;
 
   const int s_first = kmin >> 5, s_last = kmax >> 5;
-  for (int st = s_first + (split ? wave : 0); st <= s_last; st += split ? 4 : 1) {
-    const int k0 = st << 5;
+  const int n_kept = min((keep_first + 31) >> 5, s_first);         // steps of kept first tokens that lie before the window's steps
+  const int n_steps = n_kept + s_last - s_first + 1;
+  for (int si = split ? wave : 0; si < n_steps; si += split ? 4 : 1) {
+    const int k0 = (si < n_kept ? si : s_first + si - n_kept) << 5;
     const size_t pg = (size_t)table[k0 / bs] * G + g;
     const int koff = k0 % bs;
     u32x4_t kreg[2][MK];
@@ -352,7 +406,7 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
         float s = sc[hg][i] * scale;
         if (cap > 0.f) s = cap * (1.0f - 2.0f / (1.0f + __expf(2.0f * s * inv_cap)));
         s -= slope * (float)(pos - key);
-        s = (key <= pos && key >= first) ? s : -INFINITY;
+        s = (key <= pos && (key >= first || key < keep_first)) ? s : -INFINITY;
         sv[hg * 4 + i] = s;
         smax = fmaxf(smax, s);
       }
@@ -458,7 +512,15 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
         }
     }
   }
-  bf16_t* orow = out + ((size_t)token * H + head) * Dv + qd * 4;
+  if (gate) {
+    const float* gr = gate + (size_t)token * ldg + head * Dv + qd * 4;
+#pragma unroll
+    for (int i = 0; i < MV; ++i)
+      if (i < DVT)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[i][e] = acc[i][e] / (1.0f + __expf(-gr[i * 16 + e])) * out_scale;
+  }
+  bf16_t* orow = out + (size_t)token * ldo + head * Dv + qd * 4;
 #pragma unroll
   for (int i = 0; i < MV; ++i)
     if (i < DVT) {
@@ -512,23 +574,51 @@ extern "C" int ssd_winattn_store_rope(const void* qkv_rows, long ld, const void*
   return LAUNCH_OK();
 }
 
+extern "C" int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int col_off, const void* conv_w, int taps, const float* conv_state,
+                                           int C, const int32_t* state_slots, const int64_t* positions, const int32_t* cu_q, int q_per_seq,
+                                           int B, const float* qk_freqs, int rot_dims, const int32_t* slots, void* q_out, void* k_cache,
+                                           void* v_cache, int T, int H, int G, int D, int Dv, int block_size, int f32, void* stream) {
+  if (!proj_rows || !conv_w || !conv_state || !state_slots || !positions || !slots || !q_out || !k_cache || !v_cache ||
+      (rot_dims > 0 && !qk_freqs))
+    return SSD_ERR_ARG;
+  if (T <= 0 || B <= 0 || H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || block_size <= 0 || rot_dims < 0 || rot_dims > D ||
+      (rot_dims & 1) || rot_dims > 1024 || taps < 1 || taps > CONV_MAX_TAPS || (!cu_q && q_per_seq <= 0) || col_off < 0 ||
+      C < (H + G) * D + G * Dv || ld < (long)col_off + (long)(H + G) * D + (long)G * Dv)
+    return SSD_ERR_SHAPE;
+  const int items = (H + G) * (D - rot_dims / 2) + G * Dv;
+  const int ib = (items + 255) / 256;
+  const dim3 grid(T, T >= 256 ? (ib < 4 ? ib : 4) : (ib < 16 ? ib : 16));
+  if (f32)
+    hipLaunchKernelGGL(winattn_store_conv_rope_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off,
+                       (const float*)conv_w, taps, conv_state, C, state_slots, positions, cu_q, q_per_seq, B, qk_freqs, rot_dims, slots,
+                       (float*)q_out, (float*)k_cache, (float*)v_cache, H, G, D, Dv, block_size);
+  else
+    hipLaunchKernelGGL(winattn_store_conv_rope_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off,
+                       (const bf16_t*)conv_w, taps, conv_state, C, state_slots, positions, cu_q, q_per_seq, B, qk_freqs, rot_dims, slots,
+                       (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, H, G, D, Dv, block_size);
+  return LAUNCH_OK();
+}
+
 extern "C" int ssd_winattn_paged(const void* q_rows, const void* k_cache, const void* v_cache, const float* slopes, const float* sinks,
                                  const int32_t* block_tables, int max_blocks, const int64_t* positions, const int32_t* cu_q,
                                  int q_per_seq, int max_q, int B, int T, int H, int G, int D, int Dv, int block_size, int window,
-                                 float scale, float cap, const float* out_freqs, void* out_rows, int f32, void* stream) {
+                                 int keep_first, float scale, float cap, const float* out_freqs, const float* gate_rows, long ldg,
+                                 float out_scale, void* out_rows, long ldo, int f32, void* stream) {
   if (!q_rows || !k_cache || !v_cache || !block_tables || !positions || !out_rows) return SSD_ERR_ARG;
   if (T <= 0 || B <= 0 || H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || Dv > 64 * WA_MAXV || block_size <= 0 || window < 0 ||
-      max_blocks <= 0 || (!cu_q && q_per_seq <= 0) || H > 65535 || (out_freqs && (Dv & 1)))
+      max_blocks <= 0 || (!cu_q && q_per_seq <= 0) || H > 65535 || (out_freqs && (Dv & 1)) || keep_first < 0 ||
+      ldo < (long)H * Dv || (gate_rows && ldg < (long)H * Dv))
     return SSD_ERR_SHAPE;
   if (!f32 && max_q > 0 && D % 32 == 0 && D <= 256 && Dv % (out_freqs ? 32 : 16) == 0 && Dv <= 256 && block_size % 32 == 0 && G <= 65535 &&
-      B <= 65535) {
+      B <= 65535 && ldo % 4 == 0 && (uintptr_t)out_rows % 8 == 0) {
     const int R = H / G;
     const dim3 grid((unsigned)(((long)max_q * R + 63) / 64), G, B);
     const size_t lds = (4 * 16 * (size_t)Dv + 128) * sizeof(float);
 #define WIN_MFMA(MK, MV)                                                                                                            \
   hipLaunchKernelGGL((winattn_mfma_kernel<MK, MV>), grid, dim3(256), lds, (hipStream_t)stream, (const bf16_t*)q_rows,               \
                      (const bf16_t*)k_cache, (const bf16_t*)v_cache, slopes, sinks, block_tables, max_blocks, positions, cu_q,      \
-                     q_per_seq, H, G, D, Dv, block_size, window, scale, cap, out_freqs, (bf16_t*)out_rows)
+                     q_per_seq, H, G, D, Dv, block_size, window, keep_first, scale, cap, out_freqs, gate_rows, ldg, out_scale,        \
+                     (bf16_t*)out_rows, ldo)
     if (D <= 64 && Dv <= 64) WIN_MFMA(2, 4);
     else if (D <= 128 && Dv <= 128) WIN_MFMA(4, 8);
     else {
@@ -545,10 +635,11 @@ extern "C" int ssd_winattn_paged(const void* q_rows, const void* k_cache, const 
   if (f32)
     hipLaunchKernelGGL(winattn_paged_kernel<float>, dim3(T, H), dim3(256), bytes, (hipStream_t)stream, (const float*)q_rows,
                        (const float*)k_cache, (const float*)v_cache, slopes, sinks, block_tables, max_blocks, positions, cu_q, q_per_seq,
-                       B, H, G, D, Dv, block_size, window, scale, cap, out_freqs, (float*)out_rows);
+                       B, H, G, D, Dv, block_size, window, keep_first, scale, cap, out_freqs, gate_rows, ldg, out_scale, (float*)out_rows, ldo);
   else
     hipLaunchKernelGGL(winattn_paged_kernel<bf16_t>, dim3(T, H), dim3(256), bytes, (hipStream_t)stream, (const bf16_t*)q_rows,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, slopes, sinks, block_tables, max_blocks, positions, cu_q,
-                       q_per_seq, B, H, G, D, Dv, block_size, window, scale, cap, out_freqs, (bf16_t*)out_rows);
+                       q_per_seq, B, H, G, D, Dv, block_size, window, keep_first, scale, cap, out_freqs, gate_rows, ldg, out_scale,
+                       (bf16_t*)out_rows, ldo);
   return LAUNCH_OK();
 }

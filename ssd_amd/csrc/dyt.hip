@@ -84,7 +84,7 @@ parallel_tail_kernel(float* __restrict__ x, const float* __restrict__ y_mix, con
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-glu_rows_kernel(const float* __restrict__ ab, T* __restrict__ out, int F, int act) {
+glu_rows_kernel(const float* __restrict__ ab, T* __restrict__ out, long ldo, int F, int act) {
   const size_t r = blockIdx.x;
   const float* a = ab + r * 2 * F;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < F; c += 256 * gridDim.y) {
@@ -92,7 +92,7 @@ glu_rows_kernel(const float* __restrict__ ab, T* __restrict__ out, int F, int ac
     float g;
     if (act == 0) g = z * sigmoidf_(z);
     else g = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-    stf<T>(out + r * F + c, g * u);
+    stf<T>(out + r * ldo + c, g * u);
   }
 }
 
@@ -155,14 +155,14 @@ extern "C" int ssd_parallel_tail(void* x, const void* y_mix, const void* y_ff, c
   return LAUNCH_OK();
 }
 
-extern "C" int ssd_glu_rows(const void* ab_rows, void* out_rows, int rows, int F, int act, int f32, void* stream) {
+extern "C" int ssd_glu_rows(const void* ab_rows, void* out_rows, long ldo, int rows, int F, int act, int f32, void* stream) {
   if (!ab_rows || !out_rows) return SSD_ERR_ARG;
-  if (rows <= 0 || F <= 0 || act < 0 || act > 1) return SSD_ERR_SHAPE;
+  if (rows <= 0 || F <= 0 || act < 0 || act > 1 || ldo < F) return SSD_ERR_SHAPE;
   if (f32)
     hipLaunchKernelGGL(glu_rows_kernel<float>, row_grid(rows, F), dim3(256), 0, (hipStream_t)stream, (const float*)ab_rows, (float*)out_rows,
-                       F, act);
+                       ldo, F, act);
   else
     hipLaunchKernelGGL(glu_rows_kernel<bf16_t>, row_grid(rows, F), dim3(256), 0, (hipStream_t)stream, (const float*)ab_rows,
-                       (bf16_t*)out_rows, F, act);
+                       (bf16_t*)out_rows, ldo, F, act);
   return LAUNCH_OK();
 }

@@ -55,11 +55,23 @@ __device__ __forceinline__ void stage_tile(T* lds, const T* __restrict__ src, co
   }
 }
 
-// epilogue 0: fp32 rows; 1: relu(v)^2 as element-type rows; 2: element-type rows; 5: tanh(v) as element-type rows (3, 4: see glu_act)
+// epilogue 7 (ssd_gemm_rows_decay_gate): the columns of low-rank products that feed a recurrence, as fp32 rows -- columns [0, n_decay)
+// become decays exp(-rate[n] softplus(v + bias[n])), the columns after them sigmoid gates.
+struct DecayGate { const float* rate; const float* bias; int n_decay; };
+__device__ __forceinline__ float decay_gate(float v, int n, DecayGate dg) {
+  if (n >= dg.n_decay) return 1.0f / (1.0f + expf(-v));
+  const float z = v + dg.bias[n];
+  return expf(-dg.rate[n] * (z > 20.0f ? z : log1pf(expf(z))));
+}
+
+// epilogue 0: fp32 rows; 1: relu(v)^2 as element-type rows; 2: element-type rows; 5: tanh(v) as element-type rows; 7: decay_gate(v) of
+// output column n as fp32 rows (3, 4, 6: see glu_act)
 template <typename T>
-__device__ __forceinline__ void store_out(void* y, long row, long ldy, long n, float v, int epi) {
+__device__ __forceinline__ void store_out(void* y, long row, long ldy, long n, float v, int epi, DecayGate dg) {
   if (epi == 0) {
     reinterpret_cast<float*>(y)[row * ldy + n] = v;
+  } else if (epi == 7) {
+    reinterpret_cast<float*>(y)[row * ldy + n] = decay_gate(v, (int)n, dg);
   } else {
     if (epi == 1) { v = v > 0.f ? v : 0.f; v = v * v; }
     if (epi == 5) v = tanhf(v);
@@ -87,7 +99,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 gemm_rows_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __restrict__ y, int M, int N, int K, int epi,
                  const int* __restrict__ offsets, int E, const int* __restrict__ row_idx, int idx_div, bool vec_ok, long ldx, long ldy,
-                 long gsx, long gsy, GluClamp gc) {
+                 long gsx, long gsy, GluClamp gc, DecayGate dg) {
   constexpr int PAD = 16 / sizeof(T);
   constexpr int LDT = BK + PAD;
   __shared__ __attribute__((aligned(16))) T sx[BM * LDT];
@@ -146,7 +158,7 @@ gemm_rows_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __restr
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int n = n0 + nt * 16 + (lane >> 4) * 4 + r;
-          if (n < N) store_out<T>(y, m, ldy, ycol + n, acc[nt][r], epi);
+          if (n < N) store_out<T>(y, m, ldy, ycol + n, acc[nt][r], epi, dg);
         }
     }
   } else {
@@ -182,7 +194,7 @@ gemm_rows_kernel(const T* __restrict__ x, const T* __restrict__ w, void* __restr
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int n = n0 + tn + 16 * j;
-        if (n < N) store_out<T>(y, m, ldy, ycol + n, acc[i][j], epi);
+        if (n < N) store_out<T>(y, m, ldy, ycol + n, acc[i][j], epi, dg);
       }
     }
   }
@@ -199,7 +211,7 @@ template <int NW>
 __global__ void __launch_bounds__(NW * 64)
 gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ y, int M, int N, int K, int epi,
                    const int* __restrict__ offsets, const int* __restrict__ row_idx, int idx_div, long ldx, long ldy, long gsx,
-                   long gsy, GluClamp gc) {
+                   long gsy, GluClamp gc, DecayGate dg) {
   constexpr int U = 8;
   __shared__ f32x4_t red[NW * 64];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, qd = lane >> 4;
@@ -260,7 +272,7 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, v
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int n = n0 + qd * 4 + e;
-          if (n < N) store_out<bf16_t>(y, mrow, ldy, ycol + n, sum[e], epi);
+          if (n < N) store_out<bf16_t>(y, mrow, ldy, ycol + n, sum[e], epi, dg);
         }
       }
     }
@@ -272,9 +284,10 @@ constexpr int SKINNY_MAX_ROWS = 16, SKINNY_MAX_GROUPED_ROWS = 64;
 
 int launch(const void* x, const void* w, void* y, int M, int N, int K, int epi, const int* offsets, int E, const int* row_idx,
            int idx_div, int f32, void* stream, int G = 1, long ldx = 0, long gsx = 0, long ldy = 0, long gsy = 0,
-           GluClamp gc = GluClamp{nullptr, 0.f, 0.f}) {
+           GluClamp gc = GluClamp{nullptr, 0.f, 0.f}, DecayGate dg = DecayGate{nullptr, nullptr, 0}) {
   if (!x || !w || !y) return SSD_ERR_ARG;
-  if (M <= 0 || N <= 0 || K <= 0 || epi < 0 || epi > 6) return SSD_ERR_SHAPE;
+  if (M <= 0 || N <= 0 || K <= 0 || epi < 0 || epi > 7) return SSD_ERR_SHAPE;
+  if (epi == 7 && !dg.rate) return SSD_ERR_SHAPE;
   if (epi_pairs(epi) && (f32 || (N & 1))) return SSD_ERR_SHAPE;        // the paired epilogues exist in the bf16 forms only
   if (offsets && E <= 0) return SSD_ERR_SHAPE;
   if (G < 1 || G > 65535 || (G > 1 && offsets)) return SSD_ERR_SHAPE;
@@ -293,13 +306,13 @@ int launch(const void* x, const void* w, void* y, int M, int N, int K, int epi, 
     const int kt = (K + 31) / 32;
     if (wgs < 256 && kt >= 64)
       hipLaunchKernelGGL(gemm_skinny_kernel<16>, sg, dim3(1024), 0, (hipStream_t)stream, (const bf16_t*)x, (const bf16_t*)w, y, M, N, K,
-                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc);
+                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc, dg);
     else if (wgs < 1024 && kt >= 32)
       hipLaunchKernelGGL(gemm_skinny_kernel<8>, sg, dim3(512), 0, (hipStream_t)stream, (const bf16_t*)x, (const bf16_t*)w, y, M, N, K,
-                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc);
+                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc, dg);
     else
       hipLaunchKernelGGL(gemm_skinny_kernel<4>, sg, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, (const bf16_t*)w, y, M, N, K,
-                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc);
+                         epi, offsets, row_idx, id, ldx, ldy, gsx, gsy, gc, dg);
     return hipGetLastError() == hipSuccess ? SSD_OK : SSD_ERR_LAUNCH;
   }
   const int tiles_m = (M + BM - 1) / BM + (offsets ? E : 0);
@@ -308,10 +321,10 @@ int launch(const void* x, const void* w, void* y, int M, int N, int K, int epi, 
   const bool vec_ok = ((size_t)K * esz) % 16 == 0 && x_vec && ((uintptr_t)w % 16 == 0);
   if (f32)
     hipLaunchKernelGGL(gemm_rows_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, (const float*)w, y, M, N, K,
-                       epi, offsets, E, row_idx, idx_div < 1 ? 1 : idx_div, vec_ok, ldx, ldy, gsx, gsy, gc);
+                       epi, offsets, E, row_idx, idx_div < 1 ? 1 : idx_div, vec_ok, ldx, ldy, gsx, gsy, gc, dg);
   else
     hipLaunchKernelGGL(gemm_rows_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, (const bf16_t*)w, y, M, N,
-                       K, epi, offsets, E, row_idx, idx_div < 1 ? 1 : idx_div, vec_ok, ldx, ldy, gsx, gsy, gc);
+                       K, epi, offsets, E, row_idx, idx_div < 1 ? 1 : idx_div, vec_ok, ldx, ldy, gsx, gsy, gc, dg);
   return hipGetLastError() == hipSuccess ? SSD_OK : SSD_ERR_LAUNCH;
 }
 
@@ -347,4 +360,12 @@ extern "C" int ssd_gemm_rows_batched(const void* x_rows, const void* w_rows, voi
                                      long ldy, long gsy, int epilogue, int f32, void* stream) {
   if (ldx <= 0 || ldy <= 0 || gsx < 0 || gsy < 0) return SSD_ERR_SHAPE;
   return launch(x_rows, w_rows, y, M, N, K, epilogue, nullptr, 0, nullptr, 1, f32, stream, G, ldx, gsx, ldy, gsy);
+}
+
+extern "C" int ssd_gemm_rows_decay_gate(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, const float* rate,
+                                        const float* bias, int n_decay, int f32, void* stream) {
+  if (!rate || !bias) return SSD_ERR_ARG;
+  if (n_decay < 0 || n_decay > N) return SSD_ERR_SHAPE;
+  return launch(x_rows, w_rows, y, M, N, K, 7, nullptr, 0, nullptr, 1, f32, stream, 1, 0, 0, 0, 0, GluClamp{nullptr, 0.f, 0.f},
+                DecayGate{rate, bias, n_decay});
 }

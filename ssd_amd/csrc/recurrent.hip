@@ -11,12 +11,14 @@
 //  state space          ssd_ssd_scan           per head, S [N][Dv]:  S_t = exp(-exp(A_log) dt_t) S_(t-1) + dt_t B_t x_t^T,  y_t = S_t^T C_t + D x_t,
 //                                              dt_t = softplus(dt_raw + dt_bias) (no clamp); B / C shared by the heads of a group; also
 //                                              saves the slot's last taps - 1 convolution inputs
-//  output               ssd_group_gate_norm    RMS norm in `groups` equal parts of the row, a silu gate either BEFORE the norm (gate_first)
-//                                              or after it, times a weight, as GEMM-input rows
+//  output               ssd_group_gate_norm    RMS norm in `groups` equal parts of the row, a gate (silu, sigmoid, or rows that hold the
+//                                              factor itself) either BEFORE the norm (gate_first) or after it, times a weight (per column,
+//                                              or repeated every w_period columns) and a constant, as GEMM-input rows with a row stride
 // Everything that enters a recurrence is fp32: the projections' fp32 accumulators come in as fp32 rows, decays, step sizes, states and
 // sums stay fp32.  The arithmetic of a row does not depend on the portioning: per state element one multiply-add chain in token order,
 // the output a sum over the state rows in a fixed order.
 #include "common.h"
+#include "shortconv.h"
 
 namespace {
 
@@ -29,13 +31,6 @@ template <> __device__ __forceinline__ void stf<bf16_t>(bf16_t* p, float v) { *p
 
 __device__ __forceinline__ float siluf_(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplusf_(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
-
-__device__ __forceinline__ int seq_of_row(const int32_t* cu_q, int q_per_seq, int B, int t) {
-  if (!cu_q) return t / q_per_seq;
-  int lo = 0, hi = B;
-  while (hi - lo > 1) { const int mid = (lo + hi) >> 1; if (cu_q[mid] <= t) lo = mid; else hi = mid; }
-  return lo;
-}
 
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -140,46 +135,10 @@ causal_conv_silu_kernel(const float* __restrict__ proj, long ld, int col_off, in
   const long p0 = positions[row0];
   const float* st = conv_state + (size_t)state_slots[b] * (taps - 1) * C;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < C; c += 256 * gridDim.y) {
-    float acc = ldf<T>(cb + c);
-    for (int j = 0; j < taps; ++j) {
-      const int src = t - (taps - 1 - j);
-      float v;
-      if (src >= row0) {
-        v = proj[(size_t)src * ld + col_off + c];
-      } else {
-        const int k = row0 - src;                          // k tokens before the portion's first row
-        v = p0 - k >= 0 ? st[(size_t)(taps - 1 - k) * C + c] : 0.f;
-      }
-      acc = fmaf(ldf<T>(cw + (size_t)c * taps + j), v, acc);
-    }
+    const float acc = conv_at<T>(proj, ld, col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, ldf<T>(cb + c));
     out[(size_t)t * C + c] = siluf_(acc);
   }
 }
-
-constexpr int CONV_MAX_TAPS = 16;
-
-// Channels [c_begin, c_end) of the slot's saved convolution inputs: saved row i holds the input of position p0 + n - (taps - 1) + i.
-__device__ __forceinline__ void save_conv_state(const float* proj, long ld, int conv_off, int C, float* conv_state, int taps, int slot,
-                                                int row0, int row1, long p0, int c_begin, int c_end) {
-  const int n = row1 - row0, K1 = taps - 1;
-  float* st = conv_state + (size_t)slot * K1 * C;
-  for (int c = c_begin + threadIdx.x; c < c_end; c += 256) {
-    float keep[CONV_MAX_TAPS];
-#pragma unroll
-    for (int i = 0; i < CONV_MAX_TAPS; ++i) {
-      keep[i] = 0.f;
-      if (i < K1) {
-        const long rel = (long)n - K1 + i;                // position relative to the portion's first row
-        if (rel >= 0) keep[i] = proj[(size_t)(row0 + rel) * ld + conv_off + c];
-        else if (p0 + rel >= 0) keep[i] = st[(size_t)(i + n) * C + c];
-      }
-    }
-#pragma unroll
-    for (int i = 0; i < CONV_MAX_TAPS; ++i)
-      if (i < K1) st[(size_t)i * C + c] = keep[i];
-  }
-}
-
 
 __global__ void __launch_bounds__(256)
 ssd_scan_kernel(const float* __restrict__ xbc, long ldx, int x_off, int b_off, int c_off, const float* __restrict__ proj, long ld,
@@ -357,10 +316,15 @@ scan_reg_kernel(WkvArgs wa, SsdArgs sa, const int64_t* __restrict__ positions, c
   }
 }
 
+// gate activations of the output norm: silu, sigmoid, or none (the gate rows hold the factor itself)
+__device__ __forceinline__ float gate_act(float z, int act) {
+  return act == 0 ? siluf_(z) : (act == 1 ? 1.0f / (1.0f + expf(-z)) : z);
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256)
-group_gate_norm_kernel(const float* __restrict__ o, const float* __restrict__ gate, long ldg, const T* __restrict__ w, float eps,
-                       T* __restrict__ out, int N, int groups, int gate_first) {
+group_gate_norm_kernel(const float* __restrict__ o, const float* __restrict__ gate, long ldg, int act, const T* __restrict__ w, int w_period,
+                       float eps, float scale, T* __restrict__ out, long ldo, int N, int groups, int gate_first) {
   const size_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, per = N / groups;
   const float* orow = o + t * N;
@@ -368,15 +332,15 @@ group_gate_norm_kernel(const float* __restrict__ o, const float* __restrict__ ga
   for (int g = blockIdx.y * 4 + wave; g < groups; g += 4 * gridDim.y) {
     float ss = 0.f;
     for (int c = g * per + lane; c < (g + 1) * per; c += 64) {
-      const float v = gate_first ? orow[c] * siluf_(grow[c]) : orow[c];
+      const float v = gate_first ? orow[c] * gate_act(grow[c], act) : orow[c];
       ss += v * v;
     }
     ss = wave_sum(ss);
     const float r = 1.0f / sqrtf(ss / (float)per + eps);
     for (int c = g * per + lane; c < (g + 1) * per; c += 64) {
-      const float gs = siluf_(grow[c]);
-      const float v = gate_first ? orow[c] * gs * r * ldf<T>(w + c) : orow[c] * r * ldf<T>(w + c) * gs;
-      stf<T>(out + t * N + c, v);
+      const float gs = gate_act(grow[c], act), wv = ldf<T>(w + (w_period ? c % w_period : c));
+      const float v = gate_first ? orow[c] * gs * r * wv : orow[c] * r * wv * gs;
+      stf<T>(out + t * ldo + c, v * scale);
     }
   }
 }
@@ -506,17 +470,21 @@ extern "C" int ssd_ssd_scan(const void* xbc_rows, long ldx, int x_off, int b_off
   return LAUNCH_OK();
 }
 
-extern "C" int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, const void* weight, float eps, void* out_rows,
-                                   int T, int N, int groups, int gate_first, int f32, void* stream) {
+extern "C" int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, int gate_act, const void* weight, int w_period,
+                                   float eps, float out_scale, void* out_rows, long ldo, int T, int N, int groups, int gate_first, int f32,
+                                   void* stream) {
   if (!o_rows || !gate_rows || !weight || !out_rows) return SSD_ERR_ARG;
-  if (T <= 0 || N <= 0 || groups <= 0 || N % groups || ldg < N) return SSD_ERR_SHAPE;
+  if (T <= 0 || N <= 0 || groups <= 0 || N % groups || ldg < N || ldo < N || gate_act < 0 || gate_act > 2 || w_period < 0)
+    return SSD_ERR_SHAPE;
   const int gb = (groups + 3) / 4;
   const dim3 grid(T, T >= 256 ? 1 : (gb < 16 ? gb : 16));
   if (f32)
     hipLaunchKernelGGL(group_gate_norm_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows,
-                       (const float*)gate_rows, ldg, (const float*)weight, eps, (float*)out_rows, N, groups, gate_first);
+                       (const float*)gate_rows, ldg, gate_act, (const float*)weight, w_period, eps, out_scale, (float*)out_rows, ldo, N,
+                       groups, gate_first);
   else
     hipLaunchKernelGGL(group_gate_norm_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows,
-                       (const float*)gate_rows, ldg, (const bf16_t*)weight, eps, (bf16_t*)out_rows, N, groups, gate_first);
+                       (const float*)gate_rows, ldg, gate_act, (const bf16_t*)weight, w_period, eps, out_scale, (bf16_t*)out_rows, ldo, N,
+                       groups, gate_first);
   return LAUNCH_OK();
 }

@@ -43,6 +43,9 @@ def model_class(family: str):
     if family == "dosuvik":
         from ssd_amd.dosuvik import HipDosuvik
         return HipDosuvik
+    if family == "dusupel":
+        from ssd_amd.dusupel import HipDusupel
+        return HipDusupel
     return HipDecoder
 
 

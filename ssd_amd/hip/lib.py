@@ -16,7 +16,7 @@ _LIB = None
 
 c_void_p, c_int, c_long, c_float, c_int64 = C.c_void_p, C.c_int, C.c_long, C.c_float, C.c_int64
 
-ABI_VERSION = 6       # include/ssd_hip.h SSD_HIP_ABI_VERSION (tests/test_abi.py compares the two)
+ABI_VERSION = 7       # include/ssd_hip.h SSD_HIP_ABI_VERSION (tests/test_abi.py compares the two)
 
 # name -> argtypes, exactly include/ssd_hip.h (+ include/ssd_hip_tune.h)
 SIGNATURES = {
@@ -132,7 +132,7 @@ SIGNATURES = {
     "ssd_dyt_rows": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
     "ssd_parallel_tail": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_long, c_void_p, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_void_p],
-    "ssd_glu_rows": [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    "ssd_glu_rows": [c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p],
     "ssd_latent_store": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_float, c_int,
                          c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "ssd_latent_attn": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
@@ -154,7 +154,11 @@ SIGNATURES = {
     "ssd_winattn_store": [c_void_p, c_long, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                           c_int, c_void_p],
     "ssd_winattn_paged": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                          c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_int, c_void_p],
+                          c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_long, c_float, c_void_p,
+                          c_long, c_int, c_void_p],
+    "ssd_winattn_store_conv_rope": [c_void_p, c_long, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
+                                    c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                    c_int, c_void_p],
     "ssd_winattn_store_rope": [c_void_p, c_long, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                                c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ssd_moe_route_sigmoid_grouped": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -173,7 +177,19 @@ SIGNATURES = {
                              c_void_p, c_int, c_int, c_int, c_void_p],
     "ssd_ssd_scan": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                      c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
-    "ssd_group_gate_norm": [c_void_p, c_void_p, c_long, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "ssd_group_gate_norm": [c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_float, c_float, c_void_p, c_long, c_int, c_int, c_int,
+                            c_int, c_int, c_void_p],
+    "ssd_gemm_rows_decay_gate": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "ssd_delta_prep": [c_void_p, c_long, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                       c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                       c_int, c_int, c_int, c_void_p],
+    "ssd_delta_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
+                       c_int, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int, c_void_p, c_int, c_void_p],
+    "ssd_lnorm_embed": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int,
+                        c_long, c_int, c_void_p],
+    "ssd_lnorm_tail": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int,
+                       c_void_p],
+    "ssd_lnorm_rows": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p],
     "ssd_draft_advance": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int,
                           c_void_p, c_int, c_void_p],
 }
@@ -192,6 +208,7 @@ FAMILY_SOURCES = {
     "fomunex": _COMMON_ROWS + ["prenorm.hip", "attention_window.hip", "recurrent.hip"],
     "dosuvik": _COMMON_ROWS + ["postnorm.hip", "prenorm.hip", "dyt.hip", "attention_window.hip", "attention_latent.hip", "lightning.hip",
                                "recurrent.hip"],
+    "dusupel": _COMMON_ROWS + ["layernorm.hip", "dyt.hip", "attention_window.hip", "delta.hip", "recurrent.hip"],
 }
 
 

@@ -479,8 +479,8 @@ def parallel_tail(x, y_mix, T: int, W: int, f32: bool, *, y_ff=None, ydn=None, i
                                             T, W, int(f32), _stream()), "ssd_parallel_tail")
 
 
-def glu_rows(ab, out_rows, rows: int, F: int, act: int, f32: bool):
-    _check(load_library().ssd_glu_rows(_p(ab), _p(out_rows), rows, F, act, int(f32), _stream()), "ssd_glu_rows")
+def glu_rows(ab, out_rows, rows: int, F: int, act: int, f32: bool, ldo: int = 0):
+    _check(load_library().ssd_glu_rows(_p(ab), _p(out_rows), ldo or F, rows, F, act, int(f32), _stream()), "ssd_glu_rows")
 
 
 def latent_store(proj, ld: int, q_rank: int, kv_rank: int, rot: int, H: int, q_norm_w, kv_norm_w, eps: float, positions, freqs,
@@ -575,12 +575,24 @@ def winattn_store(qkv, ld: int, eps: float, slots, q_out, k_cache, v_cache, T: i
 
 def winattn_paged(q, k_cache, v_cache, slopes, sinks, block_tables, max_blocks: int, positions, B: int, T: int, H: int, G: int, D: int,
                   Dv: int, block_size: int, window: int, scale: float, cap: float, out_rows, f32: bool, cu_q=None, q_per_seq: int = 0,
-                  max_q: int = 0, out_freqs=None):
+                  max_q: int = 0, out_freqs=None, keep_first: int = 0, gate=None, ldg: int = 0, out_scale: float = 1.0, ldo: int = 0):
     """max_q > 0 (an upper bound of the rows a sequence brings; bf16, aligned head sizes, block_size % 32 == 0): the MFMA form.
-    out_freqs (fp32 [Dv / 2]): every head's output turns back by the query's position (values cached rotated by their own)."""
+    out_freqs (fp32 [Dv / 2]): every head's output turns back by the query's position (values cached rotated by their own).
+    keep_first: so many first tokens of a sequence stay visible whatever the window.  gate (fp32 rows, stride ldg): outputs times
+    sigmoid(gate) * out_scale.  ldo: row stride of out_rows (0: H * Dv)."""
     _check(load_library().ssd_winattn_paged(_p(q), _p(k_cache), _p(v_cache), _p(slopes), _p(sinks), _p(block_tables), max_blocks,
-                                            _p(positions), _p(cu_q), q_per_seq, max_q, B, T, H, G, D, Dv, block_size, window, scale, cap,
-                                            _p(out_freqs), _p(out_rows), int(f32), _stream()), "ssd_winattn_paged")
+                                            _p(positions), _p(cu_q), q_per_seq, max_q, B, T, H, G, D, Dv, block_size, window, keep_first, scale,
+                                            cap, _p(out_freqs), _p(gate), ldg, out_scale, _p(out_rows), ldo or H * Dv, int(f32), _stream()),
+           "ssd_winattn_paged")
+
+
+def winattn_store_conv_rope(proj, ld: int, col_off: int, conv_w, taps: int, conv_state, C: int, state_slots, positions, B: int, qk_freqs,
+                            rot_dims: int, slots, q_out, k_cache, v_cache, T: int, H: int, G: int, D: int, Dv: int, block_size: int,
+                            f32: bool, cu_q=None, q_per_seq: int = 0):
+    _check(load_library().ssd_winattn_store_conv_rope(_p(proj), ld, col_off, _p(conv_w), taps, _p(conv_state), C, _p(state_slots),
+                                                      _p(positions), _p(cu_q), q_per_seq, B, _p(qk_freqs), rot_dims, _p(slots), _p(q_out),
+                                                      _p(k_cache), _p(v_cache), T, H, G, D, Dv, block_size, int(f32), _stream()),
+           "ssd_winattn_store_conv_rope")
 
 
 def winattn_store_rope(qkv, ld: int, q_norm_w, k_norm_w, eps: float, positions, qk_freqs, rot_dims: int, v_freqs, slots, q_out, k_cache,
@@ -618,9 +630,13 @@ def ssd_scan(xbc, ldx: int, x_off: int, b_off: int, c_off: int, proj, ld: int, d
                                        _p(conv_state), taps, B, H, G, N, Dv, _stream()), "ssd_ssd_scan")
 
 
-def group_gate_norm(o_rows, gate_rows, ldg: int, weight, eps: float, out_rows, T: int, N: int, groups: int, gate_first: bool, f32: bool):
-    _check(load_library().ssd_group_gate_norm(_p(o_rows), _p(gate_rows), ldg, _p(weight), eps, _p(out_rows), T, N, groups,
-                                              int(gate_first), int(f32), _stream()), "ssd_group_gate_norm")
+GATE_SILU, GATE_SIGMOID, GATE_NONE = 0, 1, 2
+
+
+def group_gate_norm(o_rows, gate_rows, ldg: int, weight, eps: float, out_rows, T: int, N: int, groups: int, gate_first: bool, f32: bool,
+                    gate_act: int = GATE_SILU, w_period: int = 0, out_scale: float = 1.0, ldo: int = 0):
+    _check(load_library().ssd_group_gate_norm(_p(o_rows), _p(gate_rows), ldg, gate_act, _p(weight), w_period, eps, out_scale, _p(out_rows),
+                                              ldo or N, T, N, groups, int(gate_first), int(f32), _stream()), "ssd_group_gate_norm")
 
 
 # ---- layers that normalise a sublayer's output only, depth-weighted average, retention, grouped sigmoid router ----
@@ -662,3 +678,44 @@ def moe_route_sigmoid_grouped(logits, ld: int, correction, idx, weights, T: int,
 def gemm_rows_glu_clamp(x, w, y, M: int, N: int, K: int, limit: float, alpha: float):
     """Dense product with the clamped swish-GLU as epilogue (bf16; weight rows in (gate, up) pairs): y [M][N / 2]."""
     _check(load_library().ssd_gemm_rows_glu_clamp(_p(x), _p(w), _p(y), M, N, K, limit, alpha, _stream()), "ssd_gemm_rows_glu_clamp")
+
+
+# ---- gated delta rule over recurrent state slots, layer norms of parallel layers ----
+
+def gemm_rows_decay_gate(x, w, y, M: int, N: int, K: int, rate, bias, n_decay: int, f32: bool):
+    """y fp32: columns below n_decay = exp(-rate * softplus(z + bias)), the others sigmoid(z)."""
+    _check(load_library().ssd_gemm_rows_decay_gate(_p(x), _p(w), _p(y), M, N, K, _p(rate), _p(bias), n_decay, int(f32), _stream()),
+           "ssd_gemm_rows_decay_gate")
+
+
+def delta_prep(proj, ld: int, col_off: int, conv_w, taps: int, conv_state, C: int, conv_c0: int, state_slots, positions, B: int, b_off: int,
+               qk_rows, v_rows, scalars, T: int, H: int, G: int, D: int, Dv: int, DP: int, f32: bool, *, a_off: int = -1, rate=None, bias=None,
+               lr_off: int = 0, lr_n: int = 0, lr_out=None, ld_lr: int = 0, cu_q=None, q_per_seq: int = 0):
+    _check(load_library().ssd_delta_prep(_p(proj), ld, col_off, _p(conv_w), taps, _p(conv_state), C, conv_c0, _p(state_slots), _p(positions),
+                                         _p(cu_q), q_per_seq, B, b_off, a_off, _p(rate), _p(bias), lr_off, lr_n, _p(lr_out), ld_lr,
+                                         _p(qk_rows), _p(v_rows), _p(scalars), T, H, G, D, Dv, DP, int(f32), _stream()),
+           "ssd_delta_prep")
+
+
+def delta_scan(qk_rows, v_rows, scalars, positions, state_slots, state, out_rows, B: int, H: int, G: int, D: int, Dv: int, DP: int, proj, ld: int,
+               conv_off: int, C: int, conv_state, taps: int, *, decay=None, ldd: int = 0, cu_q=None, q_per_seq: int = 0):
+    _check(load_library().ssd_delta_scan(_p(qk_rows), _p(v_rows), _p(scalars), _p(decay), ldd, _p(positions), _p(cu_q), q_per_seq,
+                                         _p(state_slots), _p(state), _p(out_rows), B, H, G, D, Dv, DP, _p(proj), ld, conv_off, C,
+                                         _p(conv_state), taps, _stream()), "ssd_delta_scan")
+
+
+def lnorm_embed(ids, table, x_out, eps: float, T: int, W: int, f32: bool, norm1=(None, None, None), norm2=(None, None, None)):
+    """x_out = table[ids]; norm1 / norm2 = (weight, bias, out rows)."""
+    _check(load_library().ssd_lnorm_embed(_p(ids), _p(table), _p(x_out), *map(_p, norm1), *map(_p, norm2), eps, T, W, table.shape[0],
+                                          int(f32), _stream()), "ssd_lnorm_embed")
+
+
+def lnorm_tail(x, y_rows, mult: float, eps: float, T: int, W: int, f32: bool, norm1=(None, None, None), norm2=(None, None, None)):
+    """x += mult * y_rows; norm1 / norm2 = (weight, bias, out rows)."""
+    _check(load_library().ssd_lnorm_tail(_p(x), _p(y_rows), mult, *map(_p, norm1), *map(_p, norm2), eps, T, W, int(f32), _stream()),
+           "ssd_lnorm_tail")
+
+
+def lnorm_rows(x, weight, bias, out_rows, eps: float, T: int, W: int, f32: bool, gather=None):
+    _check(load_library().ssd_lnorm_rows(_p(x), _p(weight), _p(bias), _p(out_rows), _p(gather), eps, T, W, int(f32), _stream()),
+           "ssd_lnorm_rows")

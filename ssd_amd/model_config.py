@@ -101,6 +101,18 @@ PRESETS = {
 }
 
 
+def safetensors_shapes(model_dir: str) -> dict:
+    """name -> shape of every tensor under a directory, from the safetensors headers alone."""
+    import glob
+    import struct
+    shapes = {}
+    for f in sorted(glob.glob(os.path.join(model_dir, "*.safetensors"))):
+        with open(f, "rb") as fh:
+            n = struct.unpack("<Q", fh.read(8))[0]
+            shapes.update({k: v.get("shape") for k, v in json.loads(fh.read(n)).items() if k != "__metadata__"})
+    return shapes
+
+
 # --------------------------------------------------------------------------------------------------
 # Fatulix: a decoder whose config.json lists its layers one by one (own keys, not a transformers config)
 # --------------------------------------------------------------------------------------------------
@@ -463,13 +475,7 @@ class FomunexConfig:
         need = [i for i, l in enumerate(self.layers) if l.mixer.kind == "wkv" and not l.mixer.decay_rank]
         if not need and self.max_position_embeddings > 0:
             return
-        import glob
-        import struct
-        shapes = {}
-        for f in sorted(glob.glob(os.path.join(model_dir, "*.safetensors"))):
-            with open(f, "rb") as fh:
-                n = struct.unpack("<Q", fh.read(8))[0]
-                shapes.update({k: v.get("shape") for k, v in json.loads(fh.read(n)).items() if k != "__metadata__"})
+        shapes = safetensors_shapes(model_dir)
         for i in need:
             name = f"l{self.layers[i].weights_of}.mix.w1"
             if name not in shapes:
@@ -698,9 +704,178 @@ class DosuvikConfig:
         return DosuvikConfig(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers)
 
 
+# --------------------------------------------------------------------------------------------------
+# Dusupel: parallel layers with a layer norm each for mixer and feed-forward (x <- x + m (mixer(ln1 x) + ff(ln2 x))) over an fp32
+# residual; mixers are gated delta rules with a decay per key channel, or two mixers side by side (windowed attention that keeps the
+# first tokens, and a gated delta rule with a decay per head); every q / k / v channel passes a short causal convolution; a span of
+# layers may run several passes with the same weights
+# --------------------------------------------------------------------------------------------------
+@dataclass
+class GatedDelta:
+    """Gated delta rule over a recurrent fp32 [dim][vdim] state per head: S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q with
+    unit q and k (q times dim^-0.5), q / k heads shared by heads / kv_heads heads, `conv`-tap causal convolutions + silu on q, k, v.
+    channel_decay: one decay per head and key channel from a projection of rank decay_rank, the output gate sigmoid of a projection of
+    rank gate_rank (tensor shapes, not config.json keys: 0 until a checkpoint's header or the caller gives them); else one decay per head
+    and a full-rank silu gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    channel_decay: bool = True
+    decay_rank: int = 0
+    gate_rank: int = 0
+    kind: str = "delta"
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    @property
+    def padded_dim(self) -> int:
+        """Key channels of a head as the kernels lay them out (padded with zeros)."""
+        return 32 if self.dim <= 32 else -(-self.dim // 64) * 64
+
+
+@dataclass
+class ConvWindowAttention:
+    """Grouped-query attention whose q, k and v pass `conv`-tap causal convolutions over time before the rotation of q and k; a sliding
+    window (a token sees itself and the window - 1 tokens before it; 0: every earlier token) that always keeps the sequence's first
+    keep_first tokens; ordinary softmax; the concatenated heads times sigmoid(W_g h) element by element."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    keep_first: int
+    conv: int
+    rope: Rotary
+    kind: str = "attention"
+
+    @property
+    def conv_channels(self) -> int:
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+
+@dataclass
+class SideBySide:
+    """Two mixers that read the same normed row: left_scale * left + right_scale * right."""
+    left: ConvWindowAttention
+    right: GatedDelta
+    left_scale: float
+    right_scale: float
+    kind: str = "parallel"
+
+
+@dataclass
+class SiluGluMLP:
+    """Dense feed-forward W_down(silu(W_gate h) * W_up h)."""
+    ff: int
+    kind: str = "dense"
+
+
+@dataclass
+class DusupelLayer:
+    mixer: object               # GatedDelta | SideBySide
+    mlp: object                 # SiluGluMLP | None
+
+
+@dataclass
+class DusupelConfig:
+    """config.json keys: architecture, vocab, width, norm.eps, residual_mult, layers[{type, mixer{...}, mlp{kind, ff} | null}],
+    loop{start, stop, times} | null.  Layers [start, stop) run `times` passes with the same weights, each pass with cache pages / state
+    of its own."""
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: list = field(default_factory=list)
+    residual_mult: float = 1.0
+    loop_start: int = 0
+    loop_stop: int = 0
+    loop_times: int = 1
+    family: str = "dusupel"
+    max_position_embeddings: int = 1 << 20
+    tie_word_embeddings: bool = False
+
+    DELTA_TYPES = ("channel_delta", "channel_delta_2")
+
+    def runs(self) -> list[tuple[int, int]]:
+        """(layer, pass) of every layer run in execution order."""
+        a, b = self.loop_start, self.loop_stop
+        if b <= a:
+            return [(i, 0) for i in range(len(self.layers))]
+        span = [(i, ps) for ps in range(self.loop_times) for i in range(a, b)]
+        return [(i, 0) for i in range(a)] + span + [(i, 0) for i in range(b, len(self.layers))]
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.runs())
+
+    @property
+    def recurrent(self) -> bool:
+        """Every mixer keeps a per-sequence state (the delta rule's matrix, the convolutions' last inputs)."""
+        return bool(self.layers)
+
+    def to_dict(self) -> dict:
+        return asdict(self)
+
+    def complete_from_checkpoint(self, model_dir: str) -> None:
+        """Sizes that only a tensor's shape gives: the ranks of the decay and gate projections."""
+        shapes = safetensors_shapes(model_dir)
+        for i, l in enumerate(self.layers):
+            if l.mixer.kind != "delta":
+                continue
+            for attr, t in (("decay_rank", "a1"), ("gate_rank", "g1")):
+                name = f"l{i}.mix.{t}"
+                if getattr(l.mixer, attr):
+                    continue
+                if name not in shapes:
+                    raise ValueError(f"Dusupel: {name} not found under {model_dir}")
+                setattr(l.mixer, attr, int(shapes[name][0]))
+
+    @staticmethod
+    def from_json(cfg: dict) -> "DusupelConfig":
+        def delta(m, channel_decay: bool) -> GatedDelta:
+            d = GatedDelta(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), int(m.get("conv") or 1), channel_decay,
+                           int(m.get("decay_rank") or 0), int(m.get("gate_rank") or 0))
+            if d.heads % d.kv_heads or d.conv < 1:
+                raise ValueError("Dusupel: heads must be a multiple of kv_heads")
+            return d
+
+        layers = []
+        for lc in cfg["layers"]:
+            m, kind = lc["mixer"], lc["type"]
+            if kind in DusupelConfig.DELTA_TYPES:
+                mixer = delta(m, True)
+            elif kind == "parallel":
+                a = m["left"]
+                mask, r = a.get("mask") or {}, a.get("rot") or {"dims": 0, "base": 1.0}
+                left = ConvWindowAttention(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]), int(a["vdim"]),
+                                           float(a["scale"]) if a.get("scale") is not None else int(a["dim"]) ** -0.5,
+                                           int(mask.get("size") or 0), int(mask.get("keep_first") or 0), int(a.get("conv") or 1),
+                                           Rotary(int(r["dims"]), float(r["base"])))
+                if left.heads % left.kv_heads or left.rope.dims % 2 or not 0 <= left.rope.dims <= left.dim:
+                    raise ValueError("Dusupel: attention sizes do not fit")
+                mixer = SideBySide(left, delta(m["right"], False), float(m["left_scale"]), float(m["right_scale"]))
+            else:
+                raise ValueError(f"Dusupel: unknown layer type {kind!r}")
+            ml = lc.get("mlp")
+            if ml is not None and ml.get("kind", "dense") != "dense":
+                raise ValueError(f"Dusupel: unknown feed-forward kind {ml['kind']!r}")
+            layers.append(DusupelLayer(mixer, None if ml is None else SiluGluMLP(int(ml["ff"]))))
+        loop = cfg.get("loop") or {}
+        mult = cfg.get("residual_mult")
+        out = DusupelConfig(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers, 1.0 if mult is None else float(mult),
+                            int(loop.get("start", 0)), int(loop.get("stop", 0)), int(loop.get("times", 1)))
+        if not (0 <= out.loop_start and out.loop_stop <= len(layers)) or out.loop_times < 1:
+            raise ValueError("Dusupel: loop out of range")
+        return out
+
+
 # config.json "architecture" values that are read by this package's own readers (everything else goes through transformers' AutoConfig)
 ARCHITECTURES = {"Fatulix": FatulixConfig.from_json, "Zerusun": ZerusunConfig.from_json, "Fomunex": FomunexConfig.from_json,
-                 "Dosuvik": DosuvikConfig.from_json}
+                 "Dosuvik": DosuvikConfig.from_json, "Dusupel": DusupelConfig.from_json}
 
 
 def read_native_config(model_dir: str):

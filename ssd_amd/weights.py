@@ -168,6 +168,40 @@ def dosuvik_param_shapes(cfg) -> list[tuple[str, tuple[int, ...]]]:
     return out + [("final.norm", (W,)), ("head", (cfg.vocab_size, W))]
 
 
+def dusupel_param_shapes(cfg) -> list[tuple[str, tuple[int, ...]]]:
+    """Tensor names and shapes of a Dusupel checkpoint (model_config.DusupelConfig); a layer that runs several passes has its tensors
+    once."""
+    W = cfg.hidden_size
+    norm = lambda n: [(n, (W,)), (n + ".b", (W,))]
+
+    def conv_qkv(p, nq, nk, nv, taps):
+        return [t for n, c in (("q", nq), ("k", nk), ("v", nv)) for t in ((p + n, (c, W)), (p + n + ".conv", (c, taps)))]
+
+    def delta(p, m):
+        nk, nv = m.kv_heads * m.dim, m.heads * m.vdim
+        out = conv_qkv(p, nk, nk, nv, m.conv) + [(p + "b", (m.heads, W)), (p + "A_log", (m.heads,)), (p + "norm", (m.vdim,)), (p + "o", (W, nv))]
+        if not m.channel_decay:
+            return out + [(p + "a", (m.heads, W)), (p + "dt_bias", (m.heads,)), (p + "g", (nv, W))]
+        assert m.decay_rank > 0 and m.gate_rank > 0, "a channel-decay layer needs its ranks (a checkpoint's tensor shapes or GatedDelta's fields)"
+        return out + [(p + "a1", (m.decay_rank, W)), (p + "a2", (m.heads * m.dim, m.decay_rank)), (p + "dt_bias", (m.heads * m.dim,)),
+                      (p + "g1", (m.gate_rank, W)), (p + "g2", (nv, m.gate_rank))]
+
+    out = [("embed", (cfg.vocab_size, W))]
+    for i, lc in enumerate(cfg.layers):
+        p, m, ml = f"l{i}.", lc.mixer, lc.mlp
+        out += norm(p + "norm1") + (norm(p + "norm2") if ml is not None else [])
+        if m.kind == "parallel":
+            a, q = m.left, p + "mix.left."
+            nv = a.heads * a.vdim
+            out += conv_qkv(q, a.heads * a.dim, a.kv_heads * a.dim, a.kv_heads * a.vdim, a.conv) + [(q + "g", (nv, W)), (q + "o", (W, nv))]
+            out += delta(p + "mix.right.", m.right)
+        else:
+            out += delta(p + "mix.", m)
+        if ml is not None:
+            out += [(p + "mlp.gate", (ml.ff, W)), (p + "mlp.up", (ml.ff, W)), (p + "mlp.down", (W, ml.ff))]
+    return out + norm("final.norm") + [("head", (cfg.vocab_size, W))]
+
+
 def param_shapes(cfg: ModelConfig) -> list[tuple[str, tuple[int, ...]]]:
     if cfg.family == "eagle3":
         return eagle_param_shapes(cfg)
@@ -179,6 +213,8 @@ def param_shapes(cfg: ModelConfig) -> list[tuple[str, tuple[int, ...]]]:
         return fomunex_param_shapes(cfg)
     if cfg.family == "dosuvik":
         return dosuvik_param_shapes(cfg)
+    if cfg.family == "dusupel":
+        return dusupel_param_shapes(cfg)
     h, hd, nh, nkv, I, V = cfg.hidden_size, cfg.head_dim, cfg.num_heads, cfg.num_kv_heads, cfg.intermediate_size, cfg.vocab_size
     out = [("model.embed_tokens.weight", (V, h))]
     for i in range(cfg.num_layers):
@@ -393,7 +429,7 @@ def synthetic_tensor(name: str, shape, seed: int, std: float, gen_device: str, n
         return (idx - torch.arange(shape[0])).to(torch.int64).to(gen_device)
     if name.endswith(".alpha"):     # Dynamic-Tanh norms: the scalar inside the tanh; its bias is the '.b' tensor
         return torch.full(shape, 0.5, dtype=BF16, device=gen_device)
-    if name.endswith(".b"):
+    if name.endswith(".b") and len(shape) == 1:
         return torch.zeros(shape, dtype=BF16, device=gen_device)
     if "norm" in name or name.endswith("_ln.weight"):
         if norm_jitter == 0.0:
