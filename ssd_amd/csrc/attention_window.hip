@@ -143,7 +143,7 @@ winattn_store_rope_kernel(const float* __restrict__ qkv, long ld, const T* __res
 // order q | k | v), then the pair (i, i + half) of every q / k head turns by pos * qk_freqs[i].  The channels' columns start at col_off of
 // the projection rows; they are channels 0 .. of conv_state's C.  grid = (tokens, column blocks); the pairs' sines and cosines are
 // computed once per workgroup.
-template <typename T>
+template <typename T, int TAPS>
 __global__ void __launch_bounds__(256)
 winattn_store_conv_rope_kernel(const float* __restrict__ proj, long ld, int col_off, const T* __restrict__ cw, int taps,
                                const float* __restrict__ conv_state, int C, const int32_t* __restrict__ state_slots,
@@ -166,7 +166,7 @@ winattn_store_conv_rope_kernel(const float* __restrict__ proj, long ld, int col_
   const int off = slot >= 0 ? slot % bs : 0;
   const int per = D - half;                                // items of a q / k head: `half` pairs, then the entries that do not turn
   const int n_qk = (H + G) * per, n_all = n_qk + (slot >= 0 ? G * Dv : 0);
-  auto val = [&](int c) { return conv_at<T>(proj, ld, (long)col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, 0.f); };
+  auto val = [&](int c) { return conv_at<T, TAPS>(proj, ld, (long)col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, 0.f); };
   for (int u = blockIdx.y * 256 + threadIdx.x; u < n_all; u += 256 * gridDim.y) {
     if (u < n_qk) {
       const int hd = u / per, i = u % per;
@@ -587,15 +587,15 @@ extern "C" int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int c
     return SSD_ERR_SHAPE;
   const int items = (H + G) * (D - rot_dims / 2) + G * Dv;
   const int ib = (items + 255) / 256;
-  const dim3 grid(T, T >= 256 ? (ib < 4 ? ib : 4) : (ib < 16 ? ib : 16));
-  if (f32)
-    hipLaunchKernelGGL(winattn_store_conv_rope_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off,
-                       (const float*)conv_w, taps, conv_state, C, state_slots, positions, cu_q, q_per_seq, B, qk_freqs, rot_dims, slots,
-                       (float*)q_out, (float*)k_cache, (float*)v_cache, H, G, D, Dv, block_size);
-  else
-    hipLaunchKernelGGL(winattn_store_conv_rope_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off,
-                       (const bf16_t*)conv_w, taps, conv_state, C, state_slots, positions, cu_q, q_per_seq, B, qk_freqs, rot_dims, slots,
-                       (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, H, G, D, Dv, block_size);
+  const dim3 grid(T, T >= 256 ? (ib < 4 ? ib : 4) : (ib < 64 ? ib : 64));
+#define CONV_ROPE(TY, TAPS)                                                                                                              \
+  hipLaunchKernelGGL((winattn_store_conv_rope_kernel<TY, TAPS>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld,     \
+                     col_off, (const TY*)conv_w, taps, conv_state, C, state_slots, positions, cu_q, q_per_seq, B, qk_freqs, rot_dims, slots, \
+                     (TY*)q_out, (TY*)k_cache, (TY*)v_cache, H, G, D, Dv, block_size)
+#define CONV_ROPE_T(TAPS) do { if (f32) CONV_ROPE(float, TAPS); else CONV_ROPE(bf16_t, TAPS); } while (0)
+  CONV_TAPS(taps, CONV_ROPE_T);
+#undef CONV_ROPE_T
+#undef CONV_ROPE
   return LAUNCH_OK();
 }
 

@@ -35,7 +35,7 @@ struct PrepArgs {
 
 // grid = (tokens, column blocks); the work of a token is a list of wave units: one per q / k head (both vectors, their norms, their
 // product, the scalars of the heads that share them), one per 64 value channels, one per 64 copied columns.
-template <typename T>
+template <typename T, int TAPS>
 __global__ void __launch_bounds__(256)
 delta_prep_kernel(PrepArgs a, const T* __restrict__ cw, const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
                   int q_per_seq, const int32_t* __restrict__ state_slots, int B, float* __restrict__ qk, float* __restrict__ vrows,
@@ -47,7 +47,7 @@ delta_prep_kernel(PrepArgs a, const T* __restrict__ cw, const int64_t* __restric
   const long p0 = positions[row0];
   const float* st = a.conv_state + (size_t)state_slots[b] * (a.taps - 1) * a.C;
   auto val = [&](int c) {
-    return siluf_(conv_at<T>(a.proj, a.ld, (long)a.col_off + c, a.conv_c0 + c, a.C, cw + (size_t)c * a.taps, a.taps, st, t, row0, p0, 0.f));
+    return siluf_(conv_at<T, TAPS>(a.proj, a.ld, (long)a.col_off + c, a.conv_c0 + c, a.C, cw + (size_t)c * a.taps, a.taps, st, t, row0, p0, 0.f));
   };
   const int R = H / G, Nk = G * D, Nv = H * Dv;
   const int v_units = (Nv + 63) >> 6, lr_units = lr_out ? (int)((a.ld_lr + 63) >> 6) : 0;
@@ -59,7 +59,7 @@ delta_prep_kernel(PrepArgs a, const T* __restrict__ cw, const int64_t* __restric
       for (int i = 0; i < KEEP; ++i) {
         vq[i] = vk[i] = 0.f;
         const int d = lane + i * 64;
-        if (d < D) { vq[i] = val(u * D + d); vk[i] = val(Nk + u * D + d); }
+        if (i * 64 < D && d < D) { vq[i] = val(u * D + d); vk[i] = val(Nk + u * D + d); }
         sq = fmaf(vq[i], vq[i], sq);
         sk = fmaf(vk[i], vk[i], sk);
         dot = fmaf(vq[i], vk[i], dot);
@@ -175,32 +175,51 @@ delta_scan_kernel(const float4* __restrict__ qk, const float* __restrict__ vrows
     if (tid < nb) ss[tid] = rs;
     __syncthreads();
     if (r + TB < row1) fetch(r + TB);
-    for (int tt = 0; tt < nb; ++tt) {
-      const float4 sc = ss[tt];           // beta, decay of the head, <q, k>
-      const float v = sv[tt * COLS + col];
-      float4 k[NJ];
-      float4 ak{0.f, 0.f, 0.f, 0.f}, aq{0.f, 0.f, 0.f, 0.f};
+    // the staged values of a token are read one token ahead of their use: the LDS latency hides behind the current token's chain
+    float4 k[NJ], q[NJ], g[NJ], sc;
+    float v;
+    auto read = [&](int tt) {
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
         const int i = tt * D4 + P * j + p;
         k[j] = sk[i];
-        const float4 q = sq[i];
-        const float4 g = CH ? sg[i] : float4{sc.y, sc.y, sc.y, sc.y};
-        s[j].x *= g.x; s[j].y *= g.y; s[j].z *= g.z; s[j].w *= g.w;
-        ak.x = fmaf(s[j].x, k[j].x, ak.x); ak.y = fmaf(s[j].y, k[j].y, ak.y);
-        ak.z = fmaf(s[j].z, k[j].z, ak.z); ak.w = fmaf(s[j].w, k[j].w, ak.w);
-        aq.x = fmaf(s[j].x, q.x, aq.x); aq.y = fmaf(s[j].y, q.y, aq.y);
-        aq.z = fmaf(s[j].z, q.z, aq.z); aq.w = fmaf(s[j].w, q.w, aq.w);
+        q[j] = sq[i];
+        if (CH) g[j] = sg[i];
       }
-      const float dk = col_sum<P>((ak.x + ak.y) + (ak.z + ak.w));
-      const float dq = col_sum<P>((aq.x + aq.y) + (aq.z + aq.w));
-      const float u = sc.x * (v - dk);
+      sc = ss[tt];                        // beta, decay of the head, <q, k>
+      v = sv[tt * COLS + col];
+    };
+    auto step = [&](int tt) {
+      float4 kc[NJ];
+      const float beta = sc.x, gh = sc.y, kq = sc.z, vc = v;
+      float4 ak{0.f, 0.f, 0.f, 0.f}, aq{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
-        s[j].x = fmaf(k[j].x, u, s[j].x); s[j].y = fmaf(k[j].y, u, s[j].y);
-        s[j].z = fmaf(k[j].z, u, s[j].z); s[j].w = fmaf(k[j].w, u, s[j].w);
+        kc[j] = k[j];
+        const float4 gj = CH ? g[j] : float4{gh, gh, gh, gh};
+        s[j].x *= gj.x; s[j].y *= gj.y; s[j].z *= gj.z; s[j].w *= gj.w;
+        ak.x = fmaf(s[j].x, k[j].x, ak.x); ak.y = fmaf(s[j].y, k[j].y, ak.y);
+        ak.z = fmaf(s[j].z, k[j].z, ak.z); ak.w = fmaf(s[j].w, k[j].w, ak.w);
+        aq.x = fmaf(s[j].x, q[j].x, aq.x); aq.y = fmaf(s[j].y, q[j].y, aq.y);
+        aq.z = fmaf(s[j].z, q[j].z, aq.z); aq.w = fmaf(s[j].w, q[j].w, aq.w);
       }
-      if (p == 0) so[tt * COLS + col] = fmaf(u, sc.z, dq);
+      read(min(tt + 1, TB - 1));
+      const float dk = col_sum<P>((ak.x + ak.y) + (ak.z + ak.w));
+      const float dq = col_sum<P>((aq.x + aq.y) + (aq.z + aq.w));
+      const float u = beta * (vc - dk);
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        s[j].x = fmaf(kc[j].x, u, s[j].x); s[j].y = fmaf(kc[j].y, u, s[j].y);
+        s[j].z = fmaf(kc[j].z, u, s[j].z); s[j].w = fmaf(kc[j].w, u, s[j].w);
+      }
+      if (p == 0) so[tt * COLS + col] = fmaf(u, kq, dq);
+    };
+    read(0);
+    if (nb == TB) {
+#pragma unroll 4
+      for (int tt = 0; tt < TB; ++tt) step(tt);
+    } else {
+      for (int tt = 0; tt < nb; ++tt) step(tt);
     }
   }
   __syncthreads();
@@ -240,12 +259,13 @@ extern "C" int ssd_delta_prep(const void* proj_rows, long ld, int col_off, const
   const PrepArgs a{(const float*)proj_rows, ld, col_off, conv_c0, conv_state, C, taps, b_off, a_off, rate, bias, lr_off, lr_n, ld_lr};
   const int units = G + (H * Dv + 63) / 64 + (lr_out ? (int)((ld_lr + 63) / 64) : 0), ub = (units + 3) / 4;
   const dim3 grid(T, T >= 256 ? (ub < 4 ? ub : 4) : (ub < 64 ? ub : 64));
-  if (f32)
-    hipLaunchKernelGGL(delta_prep_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, a, (const float*)conv_w, positions, cu_q, q_per_seq,
-                       state_slots, B, (float*)qk_rows, (float*)v_rows, (float4*)scalars, (float*)lr_out, H, G, D, Dv, DP);
-  else
-    hipLaunchKernelGGL(delta_prep_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, a, (const bf16_t*)conv_w, positions, cu_q,
-                       q_per_seq, state_slots, B, (float*)qk_rows, (float*)v_rows, (float4*)scalars, (bf16_t*)lr_out, H, G, D, Dv, DP);
+#define PREP(TY, TAPS)                                                                                                              \
+  hipLaunchKernelGGL((delta_prep_kernel<TY, TAPS>), grid, dim3(256), 0, (hipStream_t)stream, a, (const TY*)conv_w, positions, cu_q,    \
+                     q_per_seq, state_slots, B, (float*)qk_rows, (float*)v_rows, (float4*)scalars, (TY*)lr_out, H, G, D, Dv, DP)
+#define PREP_T(TAPS) do { if (f32) PREP(float, TAPS); else PREP(bf16_t, TAPS); } while (0)
+  CONV_TAPS(taps, PREP_T);
+#undef PREP_T
+#undef PREP
   return LAUNCH_OK();
 }
 

@@ -124,7 +124,7 @@ wkv_scan_kernel(const float* __restrict__ proj, long ld, int r_off, int k_off, i
     shift_state[(size_t)slot * W + c] = ldf<T>(hn + (size_t)(row1 - 1) * W + c);
 }
 
-template <typename T>
+template <typename T, int TAPS>
 __global__ void __launch_bounds__(256)
 causal_conv_silu_kernel(const float* __restrict__ proj, long ld, int col_off, int C, const T* __restrict__ cw, const T* __restrict__ cb,
                         const float* __restrict__ conv_state, const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q,
@@ -135,7 +135,7 @@ causal_conv_silu_kernel(const float* __restrict__ proj, long ld, int col_off, in
   const long p0 = positions[row0];
   const float* st = conv_state + (size_t)state_slots[b] * (taps - 1) * C;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < C; c += 256 * gridDim.y) {
-    const float acc = conv_at<T>(proj, ld, col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, ldf<T>(cb + c));
+    const float acc = conv_at<T, TAPS>(proj, ld, col_off + c, c, C, cw + (size_t)c * taps, taps, st, t, row0, p0, ldf<T>(cb + c));
     out[(size_t)t * C + c] = siluf_(acc);
   }
 }
@@ -423,14 +423,13 @@ extern "C" int ssd_causal_conv_silu(const void* proj_rows, long ld, int col_off,
   if (T <= 0 || C <= 0 || taps < 1 || taps > CONV_MAX_TAPS || B <= 0 || (!cu_q && q_per_seq <= 0) || ld < col_off + C) return SSD_ERR_SHAPE;
   const int cb = (C + 255) / 256;
   const dim3 grid(T, cb < 64 ? cb : 64);
-  if (f32)
-    hipLaunchKernelGGL(causal_conv_silu_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off, C,
-                       (const float*)conv_w, (const float*)conv_b, conv_state, positions, cu_q, q_per_seq, state_slots, B,
-                       (float*)out_rows, taps);
-  else
-    hipLaunchKernelGGL(causal_conv_silu_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off, C,
-                       (const bf16_t*)conv_w, (const bf16_t*)conv_b, conv_state, positions, cu_q, q_per_seq, state_slots, B,
-                       (float*)out_rows, taps);
+#define CONV_SILU(TY, TAPS)                                                                                                        \
+  hipLaunchKernelGGL((causal_conv_silu_kernel<TY, TAPS>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld, col_off, C, \
+                     (const TY*)conv_w, (const TY*)conv_b, conv_state, positions, cu_q, q_per_seq, state_slots, B, (float*)out_rows, taps)
+#define CONV_SILU_T(TAPS) do { if (f32) CONV_SILU(float, TAPS); else CONV_SILU(bf16_t, TAPS); } while (0)
+  CONV_TAPS(taps, CONV_SILU_T);
+#undef CONV_SILU_T
+#undef CONV_SILU
   return LAUNCH_OK();
 }
 

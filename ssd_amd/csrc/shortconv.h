@@ -17,25 +17,42 @@ __device__ __forceinline__ int seq_of_row(const int32_t* cu_q, int q_per_seq, in
 }
 
 // Channel c of the convolution at row t of a portion that starts at row row0 / position p0, on top of `acc`.  col: the channel's column
-// in the projection rows; w: its `taps` weights; st: the slot's saved rows (row stride C).
-template <typename T>
+// in the projection rows; w: its weights; st: the slot's saved rows (row stride C).  TAPS: the tap count, or 0 for any (`taps`).  All
+// inputs are loaded before the first product (a load that must not count reads the current row's entry and is replaced by zero), so the
+// taps cost one memory round trip.
+template <typename T, int TAPS>
 __device__ __forceinline__ float conv_at(const float* __restrict__ proj, long ld, long col, int c, int C, const T* __restrict__ w, int taps,
                                          const float* __restrict__ st, int t, int row0, long p0, float acc) {
-  for (int j = 0; j < taps; ++j) {
-    const int src = t - (taps - 1 - j);
-    float v;
-    if (src >= row0) {
-      v = proj[(size_t)src * ld + col];
-    } else {
-      const int k = row0 - src;                            // k tokens before the portion's first row
-      v = p0 - k >= 0 ? st[(size_t)(taps - 1 - k) * C + c] : 0.f;
-    }
-    float wv;
-    if constexpr (sizeof(T) == 2) wv = bf2f(w[j]); else wv = w[j];
-    acc = fmaf(wv, v, acc);
+  constexpr int N = TAPS > 0 ? TAPS : CONV_MAX_TAPS;
+  const int n = TAPS > 0 ? TAPS : taps;
+  const float* cur = proj + (size_t)t * ld + col;
+  float v[N], wv[N];
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    v[j] = wv[j] = 0.f;
+    if (TAPS == 0 && j >= n) continue;
+    const int back = n - 1 - j, k = row0 - (t - back);     // k > 0: so many tokens before the portion's first row
+    const bool saved = k > 0, zero = saved && p0 - k < 0;
+    const float* src = zero ? cur : (saved ? st + (size_t)(n - 1 - k) * C + c : cur - (size_t)back * ld);
+    v[j] = *src;
+    if (zero) v[j] = 0.f;
+    if constexpr (sizeof(T) == 2) wv[j] = bf2f(w[j]); else wv[j] = w[j];
   }
+#pragma unroll
+  for (int j = 0; j < N; ++j)
+    if (TAPS > 0 || j < n) acc = fmaf(wv[j], v[j], acc);
   return acc;
 }
+// runs BODY(TAPS) with the tap count as a constant for the usual counts
+#define CONV_TAPS(taps, BODY)      \
+  do {                             \
+    switch (taps) {                \
+      case 2: BODY(2); break;      \
+      case 3: BODY(3); break;      \
+      case 4: BODY(4); break;      \
+      default: BODY(0); break;     \
+    }                              \
+  } while (0)
 
 // Channels [c_begin, c_end) of the slot's saved convolution inputs: saved row i holds the input of position p0 + n - (taps - 1) + i.
 __device__ __forceinline__ void save_conv_state(const float* proj, long ld, int conv_off, int C, float* conv_state, int taps, int slot,

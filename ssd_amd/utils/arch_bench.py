@@ -17,6 +17,9 @@ the same parameter count.
 --workload dosuvik: the Dosuvik decoder (output-norm layers with a depth average; latent attention / retention / windowed attention with
 rotated values and a sink / retention; grouped sigmoid-routed silu-GLU experts and one dense clamped GLU) beside the closest existing
 family, Zerusun (the same latent attention and linear-attention scan kernels, a grouped router, silu-GLU experts), at equal size.
+--workload dusupel: the Dusupel decoder (parallel layers; windowed attention beside a gated delta rule / gated delta rule with a decay
+per channel; dense silu GLU) beside the closest existing family, Fomunex (the same windowed attention over pages, recurrent scans with a
+short convolution over state slots, the same output norm), at equal parameter count with dense feed-forwards.
 """
 from __future__ import annotations
 
@@ -28,6 +31,7 @@ import torch
 from ssd_amd.config import Config
 from ssd_amd.engine.block_manager import BlockManager
 from ssd_amd.engine.sequence import Sequence
+from ssd_amd.model_config import ConvWindowAttention, DusupelConfig, DusupelLayer, GatedDelta, SideBySide, SiluGluMLP
 from ssd_amd.model_config import (BiasedGroupRoutedMLP, ClampedGluMLP, DosuvikConfig, DosuvikLayer, GatedLatentAttention, RetentionMixer,
                                   Rotary, RotaryWindowAttention)
 from ssd_amd.model_config import (DiffAttention, FatulixConfig, FatulixLayer, FomunexConfig, FomunexLayer, GroupRoutedMLP, LatentAttention,
@@ -93,6 +97,30 @@ def dosuvik_models(size: str):
     att = RotaryWindowAttention(Hh, G, 128, 128, 128 ** -0.5, 1024, Rotary(64, 1e4))
     layers = [DosuvikLayer(lat, moe), DosuvikLayer(ret, dense), DosuvikLayer(att, moe), DosuvikLayer(ret, moe)]
     return DosuvikConfig(VOCAB, W, 1e-5, (layers * (L // 4 + 1))[:L]), zer
+
+
+def dusupel_models(size: str):
+    """(Dusupel, Fomunex) of equal size: the same width, layers, vocabulary, attention heads and window; both feed-forwards dense, Fomunex's
+    as wide as makes the two models' parameter counts equal (its layers have lighter mixers and two-matrix feed-forwards)."""
+    from ssd_amd.weights import param_shapes
+    W, L, Hh, G, _, _, _, _, inter = SIZES[size]
+    att = ConvWindowAttention(Hh, G, 128, 128, 128 ** -0.5, 1024, 64, 4, Rotary(64, 1e6))
+    par = DusupelLayer(SideBySide(att, GatedDelta(Hh // 2, Hh // 4, 128, 128, 4, False), 0.8, 1.1), SiluGluMLP(inter))
+    dlt = DusupelLayer(GatedDelta(Hh, Hh, 128, 128, 4, True, 128, 128), SiluGluMLP(inter))
+    dus = DusupelConfig(VOCAB, W, 1e-5, ([par, dlt] * L)[:L], 0.5)
+    fatt = WindowAttention(Hh, G, 128, 128, 0.125, 30.0, 1024)
+    mixers = [fatt, Mamba2Mixer(W // 64, 64, 128, 1, 4, 1), fatt, WkvMixer(W // 64, 64, 64)]
+    fom = lambda ff: FomunexConfig(VOCAB, W, 1e-5, [FomunexLayer(m, PolyNormMLP(ff), i) for i, m in enumerate((mixers * L)[:L])], 8192, 1.0, 30.0)
+    count = lambda cfg: sum(_numel(s) for n, s in param_shapes(cfg) if n not in ("embed", "pos", "head"))
+    ff = (count(dus) - count(fom(64))) // (2 * W * L) + 64
+    return dus, fom(ff // 64 * 64)
+
+
+def _numel(shape) -> int:
+    n = 1
+    for s in shape:
+        n *= s
+    return n
 
 
 def _runner(cfg, max_len: int, batch: int, dtype: str = "bfloat16"):
@@ -222,6 +250,35 @@ def run_dosuvik(args) -> dict:
             "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
             "config": {"model": "dosuvik-w4096-synthetic", "global_batch": 8, "seq_len": prompt_len, "parallelism": "single GPU"},
             "closest_model_value": results[k]["zerusun_equal_size"]["decode_tok_s"], "sizes": results}
+
+
+def run_dusupel(args) -> dict:
+    """bench.py --workload dusupel: the Dusupel decoder beside an equal-size Fomunex decoder."""
+    sizes = list(SIZES) if args.arch_size == "all" else [args.arch_size]
+    batches = [args.arch_batch] if args.arch_batch else [1, 8]
+    only = getattr(args, "arch_only", "both")
+    prompt_len, steps, warmup = 2048, max(args.steps, 8), max(args.warmup, 2)
+    results = {}
+    for size in sizes:
+        dus, fom = dusupel_models(size)
+        for b in batches:
+            key = f"{size}_b{b}"
+            results[key] = {}
+            if only in ("both", "dusupel"):
+                results[key]["dusupel"] = measure(dus, prompt_len, b, steps, warmup)
+            if only in ("both", "fomunex"):
+                results[key]["fomunex_equal_size"] = measure(fom, prompt_len, b, steps, warmup)
+            print(f"[arch_bench] {key}: {json.dumps(results[key])}", flush=True)
+    k = "w4096_b8"
+    if k not in results or len(results[k]) < 2:
+        return {"metric": "Dusupel / equal-size Fomunex throughput (partial run)", "sizes": results}
+    return {"metric": "decode tokens/s, Dusupel w4096 (4 layers: attention beside delta rule / channel-decay delta rule, dense GLU), batch 8, "
+                      "beside an equal-size Fomunex decoder",
+            "value": results[k]["dusupel"]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
+            "ms_per_step": results[k]["dusupel"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic (random weights, random tokens)",
+            "config": {"model": "dusupel-w4096-synthetic", "global_batch": 8, "seq_len": prompt_len, "parallelism": "single GPU"},
+            "closest_model_value": results[k]["fomunex_equal_size"]["decode_tok_s"], "sizes": results}
 
 
 def run_fomunex(args) -> dict:
