@@ -190,7 +190,7 @@ ATT_CASES = [
     # f32, H, G, D, Dv, window, keep, rot, taps, bs, mfma
     (True, 4, 2, 24, 20, 16, 3, 8, 3, 16, False), (True, 3, 1, 8, 6, 33, 0, 8, 4, 8, False), (True, 2, 2, 16, 8, 1, 1, 0, 2, 16, False),
     (True, 2, 1, 12, 12, 0, 5, 6, 1, 16, False), (True, 2, 2, 10, 9, 40, 70, 10, 6, 16, False), (False, 4, 2, 24, 20, 16, 3, 8, 3, 16, False),
-    (False, 8, 2, 32, 64, 40, 20, 16, 3, 32, True), (False, 6, 1, 96, 96, 70, 33, 24, 4, 64, True), (False, 4, 4, 64, 32, 17, 64, 64, 4, 32, True),
+    (False, 8, 2, 32, 64, 40, 20, 16, 3, 32, True), (False, 5, 1, 96, 80, 70, 33, 48, 4, 64, True), (False, 4, 4, 64, 32, 17, 64, 64, 4, 32, True),
     (False, 20, 1, 128, 48, 100, 7, 32, 2, 64, True), (False, 4, 2, 160, 160, 33, 12, 40, 3, 32, True), (False, 4, 2, 32, 32, 0, 9, 32, 3, 32, True),
 ]
 
