@@ -31,7 +31,7 @@ extern "C" {
 
 /* Bumped whenever a signature or a semantic of this header changes; ssd_abi_version() returns the value the library was built
  * with, so a consumer compiled against another header can tell (tests/abi_consumer.c does). */
-#define SSD_HIP_ABI_VERSION 7
+#define SSD_HIP_ABI_VERSION 8
 
 #define SSD_OK 0
 #define SSD_ERR_SHAPE (-1)
@@ -397,6 +397,8 @@ int ssd_rows_f32_to_bf16(const void* src, void* dst, int rows, int cols, long ld
  * element-type rows; 2: element-type rows; 3 / 4 (bf16 only, N even): w rows are (gate, up) pairs -- row 2i, row 2i + 1 -- and y is
  * act(gate) * up as element-type rows [M][N / 2], act = silu (3) or tanh-form gelu (4). */
 int ssd_gemm_rows(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, int epilogue, int f32, void* stream);
+/* y = x w^T + bias (fp32 [N], added to the fp32 accumulator), fp32 rows. */
+int ssd_gemm_rows_bias(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, const float* bias, int f32, void* stream);
 /* The same product per group: sorted rows offsets[e] .. offsets[e+1]-1 (e < E) multiply by w_rows + e * N * K; row_idx (optional)
  * names the x row of sorted row r as row_idx[r] / idx_div, y rows are the sorted rows.  rows = offsets[E]'s upper bound. */
 int ssd_gemm_rows_grouped(const void* x_rows, const void* w_rows, void* y, const int32_t* offsets, int E, const int32_t* row_idx,
@@ -537,14 +539,16 @@ int ssd_moe_route_sigmoid_grouped(const float* logits, long ld, const float* cor
  * keep_first stay visible whatever the window.  gate_rows (fp32, row stride ldg, NULL: none): the output entries are multiplied by
  * sigmoid(gate_rows[t * ldg + h * Dv + d]) * out_scale.  Output rows have row stride ldo.  max_q > 0 (an upper bound of
  * the rows any sequence of the batch brings) admits the MFMA form for bf16 and D % 32 == 0, Dv % 16 == 0, block_size % 32 == 0; max_q = 0
- * or other sizes or fp32: the scalar form. */
+ * or other sizes or fp32: the scalar form.  workspace (optional, 16-byte aligned): where the MFMA form runs and max_q * H / G <= 64, the
+ * keys of a sequence are also cut over workgroups (at least 256 keys each, by window + keep_first or the table's max_blocks pages) and
+ * the slices' partial rows joined by a second launch; 16 * (Dv + 2) floats per (sequence, kv head, 16 rows, slice). */
 int ssd_winattn_store(const void* qkv_rows, long ld, float eps, const int32_t* slots, void* q_out, void* k_cache, void* v_cache, int T,
                       int H, int G, int D, int Dv, int block_size, int f32, void* stream);
 int ssd_winattn_paged(const void* q_rows, const void* k_cache, const void* v_cache, const float* slopes, const float* sinks,
                       const int32_t* block_tables, int max_blocks, const int64_t* positions, const int32_t* cu_q, int q_per_seq,
                       int max_q, int B, int T, int H, int G, int D, int Dv, int block_size, int window, int keep_first, float scale,
                       float cap, const float* out_freqs, const float* gate_rows, long ldg, float out_scale, void* out_rows, long ldo,
-                      int f32, void* stream);
+                      int f32, void* workspace, long workspace_bytes, void* stream);
 /* The store of the rotary variant: q_out = rope(q_norm_w * q / rms(q)) with the RMS over ALL H * D entries of the row's q (k alike,
  * over G * D, into the K cache); rope turns the first rot_dims entries of every head (entry i pairs with i + rot_dims / 2) by
  * positions[t] * qk_freqs[i].  v_freqs (fp32 [Dv / 2], NULL: none): every value head turns over all Dv entries by positions[t] *
@@ -553,6 +557,11 @@ int ssd_winattn_paged(const void* q_rows, const void* k_cache, const void* v_cac
 int ssd_winattn_store_rope(const void* qkv_rows, long ld, const void* q_norm_w, const void* k_norm_w, float eps, const int64_t* positions,
                            const float* qk_freqs, int rot_dims, const float* v_freqs, const int32_t* slots, void* q_out, void* k_cache,
                            void* v_cache, int T, int H, int G, int D, int Dv, int block_size, int f32, void* stream);
+/* The store of a variant with per-head norms: q_out = rope(q_norm_w * q_h / rms(q_h)) for every head, the RMS over the head's D entries,
+ * q_norm_w [D] shared by the heads (k alike with k_norm_w, into the K cache); v as it is.  G = 0: no key and value columns, no cache. */
+int ssd_winattn_store_norm_rope(const void* qkv_rows, long ld, const void* q_norm_w, const void* k_norm_w, float eps, const int64_t* positions,
+                                const float* qk_freqs, int rot_dims, const int32_t* slots, void* q_out, void* k_cache, void* v_cache, int T,
+                                int H, int G, int D, int Dv, int block_size, int f32, void* stream);
 /* The store of a variant with short causal convolutions and no norms: every channel of q, k and v (columns col_off .. of proj_rows fp32
  * [T][ld] in that order; channels 0 .. of conv_w [C][taps] and of conv_state fp32 [slots][taps - 1][C]) becomes sum_j conv_w[c][j] *
  * in[t - (taps - 1 - j)][c]; then the first rot_dims entries of every q / k head turn.  conv_state is only read. */
@@ -562,7 +571,7 @@ int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int col_off, con
                                 int T, int H, int G, int D, int Dv, int block_size, int f32, void* stream);
 
 /* Layers that normalise a sublayer's output only, with a weighted average over the depth (csrc/postnorm.hip).
- * ssd_embed_hist: x_out fp32 [T][W] = table[ids[t]] (zeros for an id outside the table), the same into hist0 (optional) and as
+ * ssd_embed_hist: x_out fp32 [T][W] = scale * table[ids[t]] (zeros for an id outside the table), the same into hist0 (optional) and as
  * element-type rows into rows_out (optional).
  * ssd_postnorm_tail: v = y_rows[t] (fp32) or sum_j weights[t * top + j] * ydn_rows[inv[t * top + j]];  x[t] += post_weight * v /
  * sqrt(mean(v^2) + eps) (post_weight fp32 [W]).  hist (optional, fp32 levels of hist_stride floats): level hist_levels - 1 receives
@@ -572,8 +581,8 @@ int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int col_off, con
  * the first rot_dims entries of a head turn (entry i pairs with i + rot_dims / 2) by positions[t] * freqs[i], then the head is
  * multiplied by the block's scale.
  * ssd_gate_rows: out_rows[t][c] = o_rows[t * ldo + c] * sigmoid(gate_rows[t * ldg + c]) for c < N, element-type rows out. */
-int ssd_embed_hist(const int64_t* ids, const void* table, void* x_out, void* hist0, void* rows_out, int T, int W, long vocab, int f32,
-                   void* stream);
+int ssd_embed_hist(const int64_t* ids, const void* table, void* x_out, void* hist0, void* rows_out, float scale, int T, int W, long vocab,
+                   int f32, void* stream);
 int ssd_postnorm_tail(const void* y_rows, const void* ydn_rows, const int32_t* inv, const float* weights, int top,
                       const float* post_weight, float eps, void* x, void* hist, long hist_stride, int hist_levels, const float* coef,
                       void* next_out, int T, int W, int f32, void* stream);
@@ -598,7 +607,8 @@ int ssd_gate_rows(const void* o_rows, long ldo, const void* gate_rows, long ldg,
  * conv_state[slot].
  * ssd_group_gate_norm: rows of N entries in `groups` equal parts, g = act(gate_rows[t][c]) (fp32, row stride ldg; gate_act 0: silu, 1:
  * sigmoid, 2: the entry itself): out_scale * (gate_first ? weight * rms_part(o * g) : weight * rms_part(o) * g), element-type rows of
- * stride ldo; w_period > 0: weight holds w_period entries, repeated along the row. */
+ * stride ldo; w_period > 0: weight holds w_period entries, repeated along the row.  den_rows (fp32 [T][groups], NULL: none): part j of o is
+ * divided by den_rows[t][j] first. */
 int ssd_token_shift_mix(const void* hn_rows, const void* mu, const float* shift_state, const int64_t* positions, const int32_t* cu_q,
                         int q_per_seq, const int32_t* state_slots, int B, void* out_rows, int T, int W, int S, int f32, void* stream);
 int ssd_wkv_scan(const void* proj_rows, long ld, int r_off, int k_off, int v_off, const void* decay_rows, long ldw, const float* w0,
@@ -611,8 +621,8 @@ int ssd_ssd_scan(const void* xbc_rows, long ldx, int x_off, int b_off, int c_off
                  const float* dt_bias, const float* a_log, const float* skip, const int64_t* positions, const int32_t* cu_q,
                  int q_per_seq, const int32_t* state_slots, void* state, void* out_rows, int conv_off, int C, void* conv_state,
                  int taps, int B, int H, int G, int N, int Dv, void* stream);
-int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, int gate_act, const void* weight, int w_period, float eps,
-                        float out_scale, void* out_rows, long ldo, int T, int N, int groups, int gate_first, int f32, void* stream);
+int ssd_group_gate_norm(const void* o_rows, const float* den_rows, const void* gate_rows, long ldg, int gate_act, const void* weight,
+                        int w_period, float eps, float out_scale, void* out_rows, long ldo, int T, int N, int groups, int gate_first, int f32, void* stream);
 
 /* Gated delta rule over per-sequence state slots (csrc/delta.hip): per head h (q / k head h / (H / G)) over a state of D key channels x
  * Dv value columns, S <- decay S (decay: one number per head, or one per key channel), u = beta (v - S^T k), S <- S + k u^T,
@@ -635,16 +645,38 @@ int ssd_delta_scan(const void* qk_rows, const void* v_rows, const void* scalars,
                    int B, int H, int G, int D, int Dv, int DP, const void* proj_rows, long ld, int conv_off, int C, void* conv_state,
                    int taps, void* stream);
 
+/* Linear attention over an outer-product memory with a decay per head and token (csrc/memory_scan.hip): S = a S + b k v^T,
+ * o = q_scale * S^T q over state fp32 [slots][H][columns][DP], transposed, key channels padded with zeros to DP = 32 (D <= 32) or the next
+ * multiple of 64 (D <= 512); zero when a sequence's first row has position 0.  proj_rows fp32 [T][ld] holds q (H*D) at q_off, k (H*D) at
+ * k_off, v (H*Dv) at v_off; out fp32 [T][H*Dv].
+ *   decay (fp32 [H]) given: a = decay[h], b = 1; columns = Dv; m_state and den_rows are not used.
+ *   else exponential gates: i = cap tanh((proj_rows[t][i_off + h] + bias_i[h]) / cap), f = log sigmoid(cap tanh((proj_rows[t][f_off + h] +
+ *   bias_f[h]) / cap)), m' = max(f + m, i) (m = 0 before position 0), a = exp(f + m - m'), b = exp(i - m'); columns = Dv + 1, the last
+ *   one holding the normaliser n = a n + b k; den_rows fp32 [T][H] = max(|q_scale <n, q>|, exp(-m')) + 1e-6 (out is NOT divided).  m_state
+ *   fp32 [slots][H][Dv + 1]: copies of m.  gates (float4 [T][H] = a, b, exp(-m'), 0) from ssd_memory_gates over the same rows, which then
+ *   also advances m_state; NULL: computed inside the scan (the same bits). */
+int ssd_memory_gates(const void* proj_rows, long ld, int i_off, int f_off, const float* bias_i, const float* bias_f, float cap,
+                     const int64_t* positions, const int32_t* cu_q, int q_per_seq, const int32_t* state_slots, void* m_state, void* gates,
+                     int B, int H, int Dv, void* stream);
+int ssd_memory_scan(const void* proj_rows, long ld, int q_off, int k_off, int v_off, float q_scale, const float* decay, const void* gates,
+                    int i_off, int f_off, const float* bias_i, const float* bias_f, float cap, const int64_t* positions, const int32_t* cu_q,
+                    int q_per_seq, const int32_t* state_slots, void* state, void* m_state, void* out_rows, void* den_rows, int B, int H,
+                    int D, int Dv, int DP, void* stream);
+
 /* Layer norm over an fp32 residual with one or two weight sets per statistic (csrc/layernorm.hip): out = (x - mean) / sqrt(var + eps) *
  * w + b as element-type rows; out1 / out2 may be NULL (out2 only with out1).
  * ssd_lnorm_embed: x_out fp32 [T][W] = table[ids[t]] (zeros for an id outside the table) first; ssd_lnorm_tail: x += mult * y_rows
- * (fp32) first; ssd_lnorm_rows: out_rows[r] = the norm of x[gather[r]] (or x[r]). */
+ * (fp32) first; ssd_lnorm_rows: out_rows[r] = the norm of x[gather[r]] (or x[r]), bias optional.
+ * ssd_lnorm_post_tail (layers that norm a sublayer's output): x += (v - mean) / sqrt(var + eps) * weight for v = y_rows (fp32), or, y2_rows
+ * given, v = pair_scale * (w1 * y / rms(y) + w2 * y2 / rms(y2)); next_out (optional): x as element-type rows. */
 int ssd_lnorm_embed(const int64_t* ids, const void* table, void* x_out, const void* w1, const void* b1, void* out1, const void* w2,
                     const void* b2, void* out2, float eps, int T, int W, long vocab, int f32, void* stream);
 int ssd_lnorm_tail(void* x, const void* y_rows, float mult, const void* w1, const void* b1, void* out1, const void* w2, const void* b2,
                    void* out2, float eps, int T, int W, int f32, void* stream);
 int ssd_lnorm_rows(const void* x, const void* weight, const void* bias, void* out_rows, const int32_t* gather, float eps, int T, int W,
                    int f32, void* stream);
+int ssd_lnorm_post_tail(void* x, const void* y_rows, const void* y2_rows, const void* w1, const void* w2, float pair_scale,
+                        const void* weight, float eps, void* next_out, int T, int W, int f32, void* stream);
 
 /* hipGraph capture for a host that is not PyTorch -- the reference captures its decode / verify / glue / tree steps with
  * torch.cuda.CUDAGraph (ssd/engine/helpers/cudagraph_helpers.py:20-120); every entry point above only enqueues on `stream`, so the calls

@@ -20,6 +20,9 @@
 //                         relative positions.  Pairs are (i, i + n / 2) throughout.
 //   * ssd_winattn_store_conv_rope  the store of a variant without norms: a short causal convolution over time on every channel of q, k and
 //                         v (the inputs of earlier tokens from the sequence's slot), then rotary positions on q and k.
+//   * ssd_winattn_store_norm_rope  the store of a variant whose q and k are normed PER HEAD (RMS, one weight vector shared by the heads)
+//                         before the rotation; G = 0: queries only (a layer that reads another layer's pages)
+//   A decode batch may cut the keys over the grid: ssd_winattn_paged with a workspace, see the MFMA form below.
 //   keep_first > 0: the sequence's first keep_first tokens stay visible whatever the window (they keep their true positions); the walk
 //   then starts with those of them that lie before the window.  gate (fp32 rows, one entry per output entry): the heads' outputs are
 //   multiplied by sigmoid(gate) * out_scale; the output rows have a row stride.
@@ -188,6 +191,53 @@ winattn_store_conv_rope_kernel(const float* __restrict__ proj, long ld, int col_
   }
 }
 
+// Per head: x' = w * x / rms(x) over the head's D entries (one weight vector for all q heads, one for all k heads), then the pair (i, i + half)
+// turns by pos * qk_freqs[i].  One wave per head vector, the pairs' sines and cosines once per workgroup.  G = 0: no keys and values.
+template <typename T>
+__global__ void __launch_bounds__(256)
+winattn_store_norm_rope_kernel(const float* __restrict__ qkv, long ld, const T* __restrict__ wq, const T* __restrict__ wk, float eps,
+                               const int64_t* __restrict__ positions, const float* __restrict__ qk_freqs, int rot_dims,
+                               const int32_t* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ kc, T* __restrict__ vc, int H, int G,
+                               int D, int Dv, int bs) {
+  __shared__ float sn[512], cs[512];
+  const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int half = rot_dims >> 1, per = D - half;          // items of a head: `half` pairs, then the entries that do not turn
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < half; i += 256) sincosf(pos * qk_freqs[i], &sn[i], &cs[i]);
+  __syncthreads();
+  const float* row = qkv + (size_t)t * ld;
+  const int slot = G > 0 ? slots[t] : -1;
+  const long blk = slot >= 0 ? slot / bs : 0;
+  const int off = slot >= 0 ? slot % bs : 0;
+  for (int u = blockIdx.y * 4 + wave; u < H + G; u += 4 * gridDim.y) {
+    const bool isq = u < H;
+    if (!isq && slot < 0) continue;
+    const float* src = row + (size_t)u * D;                // k heads follow the q heads in the row
+    const T* w = isq ? wq : wk;
+    T* dst = isq ? q_out + ((size_t)t * H + u) * D : kc + (((size_t)blk * G + (u - H)) * bs + off) * D;
+    float ss = 0.f;
+    for (int d = lane; d < D; d += 64) { const float v = src[d]; ss += v * v; }
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+    for (int i = lane; i < per; i += 64) {
+      const float b = src[i + half] * r * ldf<T>(w + i + half);
+      if (i < half) {
+        const float a = src[i] * r * ldf<T>(w + i);
+        stf<T>(dst + i, a * cs[i] - b * sn[i]);
+        stf<T>(dst + i + half, b * cs[i] + a * sn[i]);
+      } else {
+        stf<T>(dst + i + half, b);
+      }
+    }
+  }
+  if (slot >= 0) {
+    const float* v = row + (size_t)(H + G) * D;
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < G * Dv; c += 256 * gridDim.y) {
+      const int g = c / Dv, d = c % Dv;
+      stf<T>(vc + (((size_t)blk * G + g) * Dv + d) * bs + off, v[c]);
+    }
+  }
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256)
 winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc, const float* __restrict__ slopes,
@@ -306,6 +356,10 @@ winattn_paged_kernel(const T* __restrict__ q, const T* __restrict__ kc, const T*
 //            window start of its first row to the position of its last.
 // split mode (<= 16 rows: decoding): the 4 waves share the rows and take the steps round-robin; partial (max, sum, O) meet in LDS and
 //            are merged in wave order.  The window bounds the steps, so the keys are not cut over the grid.
+// decode launch (dtiles > 0; the caller gives a workspace and no sequence brings more than 64 rows): blockIdx.x = slice * dtiles + tile;
+//            every workgroup works as in split mode on 16 rows, and the steps are dealt out to the slices as well.  With more than one
+//            slice the partial rows go to the workspace, `part` [(b * G + g) * dtiles + tile][slice][16][Dv + 2] = sums, max, sum of
+//            weights, and winattn_merge_kernel joins them in slice order: a long context of few sequences fills the chip.
 // V of keys past the last row's position is zeroed (a weight of zero times whatever an unwritten slot holds must stay zero).
 // The sink joins the denominator at the end.  The cap's tanh is 1 - 2 / (1 + exp(2x)) on the fast exponential.
 // ---------------------------------------------------------------------------------------------------------------------
@@ -315,16 +369,19 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
                     const float* __restrict__ slopes, const float* __restrict__ sinks, const int32_t* __restrict__ bt, int max_blocks,
                     const int64_t* __restrict__ positions, const int32_t* __restrict__ cu_q, int q_per_seq, int H, int G, int D, int Dv,
                     int bs, int window, int keep_first, float scale, float cap, const float* __restrict__ out_freqs,
-                    const float* __restrict__ gate, long ldg, float out_scale, bf16_t* __restrict__ out, long ldo) {
+                    const float* __restrict__ gate, long ldg, float out_scale, bf16_t* __restrict__ out, long ldo, int dtiles,
+                    float* __restrict__ part) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, qd = lane >> 4;
   const int b = blockIdx.z, g = blockIdx.y, R = H / G;
   const int KS = D >> 5, DVT = Dv >> 4;
   const int tok0 = cu_q ? cu_q[b] : b * q_per_seq;
   const int nrows = (cu_q ? cu_q[b + 1] - tok0 : q_per_seq) * R;
-  const bool split = nrows <= 16;
-  if ((int)blockIdx.x * 64 >= nrows) return;
-  const int row0 = split ? 0 : blockIdx.x * 64 + wave * 16;
+  const bool split = dtiles > 0 || nrows <= 16;
+  const int tile = dtiles > 0 ? blockIdx.x % dtiles : 0, slice = dtiles > 0 ? blockIdx.x / dtiles : 0;
+  const int slices = dtiles > 0 ? gridDim.x / dtiles : 1;
+  if ((dtiles > 0 ? tile * 16 : (int)blockIdx.x * 64) >= nrows) return;
+  const int row0 = split ? tile * 16 : blockIdx.x * 64 + wave * 16;
   if (!split && row0 >= nrows) return;                 // (tile mode has no workgroup barriers)
   const int row = row0 + r;
   const bool valid = row < nrows;
@@ -354,7 +411,7 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
   const int s_first = kmin >> 5, s_last = kmax >> 5;
   const int n_kept = min((keep_first + 31) >> 5, s_first);         // steps of kept first tokens that lie before the window's steps
   const int n_steps = n_kept + s_last - s_first + 1;
-  for (int si = split ? wave : 0; si < n_steps; si += split ? 4 : 1) {
+  for (int si = split ? slice * 4 + wave : 0; si < n_steps; si += split ? 4 * slices : 1) {
     const int k0 = (si < n_kept ? si : s_first + si - n_kept) << 5;
     const size_t pg = (size_t)table[k0 / bs] * G + g;
     const int koff = k0 % bs;
@@ -466,6 +523,16 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
           acc[i][e] = o;
         }
     mx = M; ls = L;
+    if (slices > 1) {
+      float* pr = part + (((((size_t)b * G + g) * dtiles + tile) * slices + slice) * 16 + r) * (Dv + 2);
+#pragma unroll
+      for (int i = 0; i < MV; ++i)
+        if (i < DVT)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) pr[i * 16 + qd * 4 + e] = acc[i][e];
+      if (qd == 0) { pr[Dv] = mx; pr[Dv + 1] = ls; }
+      return;
+    }
   }
   if (!valid) return;
   const float sink = sinks ? sinks[head] : -INFINITY;
@@ -531,6 +598,47 @@ winattn_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc,
     }
 }
 
+// One wave per row of the decode launch: the slices' partial rows in slice order, the sink, the output's turn, the gate.
+__global__ void __launch_bounds__(256)
+winattn_merge_kernel(const float* __restrict__ part, const float* __restrict__ sinks, const int64_t* __restrict__ positions,
+                     const int32_t* __restrict__ cu_q, int q_per_seq, int H, int G, int Dv, const float* __restrict__ out_freqs,
+                     const float* __restrict__ gate, long ldg, float out_scale, bf16_t* __restrict__ out, long ldo, int dtiles, int slices) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, R = H / G;
+  const int b = blockIdx.z, g = blockIdx.y, row = blockIdx.x * 4 + wave;
+  const int tok0 = cu_q ? cu_q[b] : b * q_per_seq;
+  const int nrows = (cu_q ? cu_q[b + 1] - tok0 : q_per_seq) * R;
+  if (row >= nrows) return;
+  const int token = tok0 + row / R, head = g * R + row % R, stride = 16 * (Dv + 2);
+  const float* pr = part + ((((size_t)b * G + g) * dtiles + (row >> 4)) * slices * 16 + (row & 15)) * (Dv + 2);
+  const float sink = sinks ? sinks[head] : -INFINITY;
+  float M = sink;
+  for (int s = lane; s < slices; s += 64) M = fmaxf(M, pr[(size_t)s * stride + Dv]);
+  M = wave_max(M);
+  float L = sinks ? __expf(sink - M) : 0.f;
+  for (int s = 0; s < slices; ++s) {
+    const float l = pr[(size_t)s * stride + Dv + 1];
+    if (l > 0.f) L = fmaf(l, __expf(pr[(size_t)s * stride + Dv] - M), L);
+  }
+  auto column = [&](int d) {
+    float o = 0.f;
+    for (int s = 0; s < slices; ++s)
+      if (pr[(size_t)s * stride + Dv + 1] > 0.f) o = fmaf(pr[(size_t)s * stride + d], __expf(pr[(size_t)s * stride + Dv] - M), o);
+    return o / L;
+  };
+  const int hv = Dv >> 1;
+  for (int d = lane; d < Dv; d += 64) {
+    float v = column(d);
+    if (out_freqs) {
+      const float o = column(d < hv ? d + hv : d - hv);
+      float sn, c;
+      sincosf((float)positions[token] * out_freqs[d < hv ? d : d - hv], &sn, &c);
+      v = d < hv ? v * c + o * sn : v * c - o * sn;
+    }
+    if (gate) v = v / (1.0f + __expf(-gate[(size_t)token * ldg + head * Dv + d])) * out_scale;
+    stf<bf16_t>(out + (size_t)token * ldo + head * Dv + d, v);
+  }
+}
+
 }  // namespace
 
 #define LAUNCH_OK() (hipGetLastError() == hipSuccess ? SSD_OK : SSD_ERR_LAUNCH)
@@ -574,6 +682,28 @@ extern "C" int ssd_winattn_store_rope(const void* qkv_rows, long ld, const void*
   return LAUNCH_OK();
 }
 
+extern "C" int ssd_winattn_store_norm_rope(const void* qkv_rows, long ld, const void* q_norm_w, const void* k_norm_w, float eps,
+                                           const int64_t* positions, const float* qk_freqs, int rot_dims, const int32_t* slots, void* q_out,
+                                           void* k_cache, void* v_cache, int T, int H, int G, int D, int Dv, int block_size, int f32,
+                                           void* stream) {
+  if (!qkv_rows || !q_norm_w || !positions || !q_out || (rot_dims > 0 && !qk_freqs)) return SSD_ERR_ARG;
+  if (G > 0 && (!k_norm_w || !slots || !k_cache || !v_cache)) return SSD_ERR_ARG;
+  if (T <= 0 || H <= 0 || G < 0 || D <= 0 || (G > 0 && (Dv <= 0 || block_size <= 0)) || rot_dims < 0 || rot_dims > D || (rot_dims & 1) ||
+      rot_dims > 1024 || ld < (long)(H + G) * D + (long)G * Dv)
+    return SSD_ERR_SHAPE;
+  const int units = (H + G + 3) / 4;
+  const dim3 grid(T, T >= 256 ? 1 : (units < 16 ? units : 16));
+  if (f32)
+    hipLaunchKernelGGL(winattn_store_norm_rope_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)qkv_rows, ld,
+                       (const float*)q_norm_w, (const float*)k_norm_w, eps, positions, qk_freqs, rot_dims, slots, (float*)q_out,
+                       (float*)k_cache, (float*)v_cache, H, G, D, Dv, block_size);
+  else
+    hipLaunchKernelGGL(winattn_store_norm_rope_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)qkv_rows, ld,
+                       (const bf16_t*)q_norm_w, (const bf16_t*)k_norm_w, eps, positions, qk_freqs, rot_dims, slots, (bf16_t*)q_out,
+                       (bf16_t*)k_cache, (bf16_t*)v_cache, H, G, D, Dv, block_size);
+  return LAUNCH_OK();
+}
+
 extern "C" int ssd_winattn_store_conv_rope(const void* proj_rows, long ld, int col_off, const void* conv_w, int taps, const float* conv_state,
                                            int C, const int32_t* state_slots, const int64_t* positions, const int32_t* cu_q, int q_per_seq,
                                            int B, const float* qk_freqs, int rot_dims, const int32_t* slots, void* q_out, void* k_cache,
@@ -603,7 +733,7 @@ extern "C" int ssd_winattn_paged(const void* q_rows, const void* k_cache, const 
                                  const int32_t* block_tables, int max_blocks, const int64_t* positions, const int32_t* cu_q,
                                  int q_per_seq, int max_q, int B, int T, int H, int G, int D, int Dv, int block_size, int window,
                                  int keep_first, float scale, float cap, const float* out_freqs, const float* gate_rows, long ldg,
-                                 float out_scale, void* out_rows, long ldo, int f32, void* stream) {
+                                 float out_scale, void* out_rows, long ldo, int f32, void* workspace, long workspace_bytes, void* stream) {
   if (!q_rows || !k_cache || !v_cache || !block_tables || !positions || !out_rows) return SSD_ERR_ARG;
   if (T <= 0 || B <= 0 || H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || Dv > 64 * WA_MAXV || block_size <= 0 || window < 0 ||
       max_blocks <= 0 || (!cu_q && q_per_seq <= 0) || H > 65535 || (out_freqs && (Dv & 1)) || keep_first < 0 ||
@@ -612,13 +742,25 @@ extern "C" int ssd_winattn_paged(const void* q_rows, const void* k_cache, const 
   if (!f32 && max_q > 0 && D % 32 == 0 && D <= 256 && Dv % (out_freqs ? 32 : 16) == 0 && Dv <= 256 && block_size % 32 == 0 && G <= 65535 &&
       B <= 65535 && ldo % 4 == 0 && (uintptr_t)out_rows % 8 == 0) {
     const int R = H / G;
-    const dim3 grid((unsigned)(((long)max_q * R + 63) / 64), G, B);
+    dim3 grid((unsigned)(((long)max_q * R + 63) / 64), G, B);
+    int dtiles = 0, slices = 1;
+    if (workspace && (long)max_q * R <= 64) {          // decode: cut the keys over the grid when the rows alone do not fill the chip
+      dtiles = (int)(((long)max_q * R + 15) / 16);
+      const long keys = window > 0 ? (long)window + keep_first : (long)max_blocks * block_size;       // an upper bound of a row's keys
+      const long rows = (long)B * G * dtiles, tile_bytes = 16L * (Dv + 2) * (long)sizeof(float);
+      long s = (512 + rows - 1) / rows;
+      s = s < (keys + 255) / 256 ? s : (keys + 255) / 256;                                            // at least 256 keys a slice
+      s = s < 64 ? s : 64;
+      s = s < workspace_bytes / (rows * tile_bytes) ? s : workspace_bytes / (rows * tile_bytes);
+      slices = s < 1 ? 1 : (int)s;
+      grid.x = (unsigned)(dtiles * slices);
+    }
     const size_t lds = (4 * 16 * (size_t)Dv + 128) * sizeof(float);
 #define WIN_MFMA(MK, MV)                                                                                                            \
   hipLaunchKernelGGL((winattn_mfma_kernel<MK, MV>), grid, dim3(256), lds, (hipStream_t)stream, (const bf16_t*)q_rows,               \
                      (const bf16_t*)k_cache, (const bf16_t*)v_cache, slopes, sinks, block_tables, max_blocks, positions, cu_q,      \
                      q_per_seq, H, G, D, Dv, block_size, window, keep_first, scale, cap, out_freqs, gate_rows, ldg, out_scale,        \
-                     (bf16_t*)out_rows, ldo)
+                     (bf16_t*)out_rows, ldo, dtiles, (float*)workspace)
     if (D <= 64 && Dv <= 64) WIN_MFMA(2, 4);
     else if (D <= 128 && Dv <= 128) WIN_MFMA(4, 8);
     else {
@@ -628,6 +770,10 @@ extern "C" int ssd_winattn_paged(const void* q_rows, const void* k_cache, const 
       WIN_MFMA(8, 16);
     }
 #undef WIN_MFMA
+    if (slices > 1)
+      hipLaunchKernelGGL(winattn_merge_kernel, dim3((unsigned)(((long)max_q * R + 3) / 4), G, B), dim3(256), 0, (hipStream_t)stream,
+                         (const float*)workspace, sinks, positions, cu_q, q_per_seq, H, G, Dv, out_freqs, gate_rows, ldg, out_scale,
+                         (bf16_t*)out_rows, ldo, dtiles, slices);
     return LAUNCH_OK();
   }
   const size_t bytes = ((size_t)D + (D & 1) + 4 * 64 + 2 * 4 * 64 + 4 * (size_t)Dv + 8) * sizeof(float);

@@ -69,6 +69,20 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+template <int CTRL>
+__device__ __forceinline__ float dpp_add(float v) {
+  return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xF, 0xF, true));
+}
+// sum over P = 8 or 16 neighbouring lanes (aligned), in every one of them: quads (xor 1, xor 2), halves of a row (mirror in 8), rows of 16 (mirror)
+template <int P>
+__device__ __forceinline__ float col_sum(float v) {
+  v = dpp_add<0xB1>(v);
+  v = dpp_add<0x4E>(v);
+  v = dpp_add<0x141>(v);
+  if constexpr (P == 16) v = dpp_add<0x140>(v);
+  return v;
+}
+
 // Threads per row of the RMSNorm kernels (norm.hip rmsnorm_kernel and comm.hip allreduce_add_rmsnorm_kernel MUST agree: the
 // chunk -> thread mapping fixes the fp32 summation order, and the fused all-reduce + norm is bit-identical to the unfused
 // pair).  A row is a latency chain (load, reduce, scale, store): hidden sizes >= 4096 get 1024 threads, i.e. at most two

@@ -87,20 +87,6 @@ delta_prep_kernel(PrepArgs a, const T* __restrict__ cw, const int64_t* __restric
   }
 }
 
-template <int CTRL>
-__device__ __forceinline__ float dpp_add(float v) {
-  return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xF, 0xF, true));
-}
-// sum over the P lanes of a column, in every one of them: quads (xor 1, xor 2), halves of a row (mirror in 8), rows of 16 (mirror)
-template <int P>
-__device__ __forceinline__ float col_sum(float v) {
-  v = dpp_add<0xB1>(v);
-  v = dpp_add<0x4E>(v);
-  v = dpp_add<0x141>(v);
-  if constexpr (P == 16) v = dpp_add<0x140>(v);
-  return v;
-}
-
 struct ConvSave { const float* proj; long ld; int off, C; float* state; int taps; };
 
 template <int P, int NJ, int TB, bool CH>

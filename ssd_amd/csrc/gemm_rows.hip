@@ -57,6 +57,7 @@ __device__ __forceinline__ void stage_tile(T* lds, const T* __restrict__ src, co
 
 // epilogue 7 (ssd_gemm_rows_decay_gate): the columns of low-rank products that feed a recurrence, as fp32 rows -- columns [0, n_decay)
 // become decays exp(-rate[n] softplus(v + bias[n])), the columns after them sigmoid gates.
+// epilogue 8 (ssd_gemm_rows_bias): fp32 rows v + bias[n].
 struct DecayGate { const float* rate; const float* bias; int n_decay; };
 __device__ __forceinline__ float decay_gate(float v, int n, DecayGate dg) {
   if (n >= dg.n_decay) return 1.0f / (1.0f + expf(-v));
@@ -65,13 +66,15 @@ __device__ __forceinline__ float decay_gate(float v, int n, DecayGate dg) {
 }
 
 // epilogue 0: fp32 rows; 1: relu(v)^2 as element-type rows; 2: element-type rows; 5: tanh(v) as element-type rows; 7: decay_gate(v) of
-// output column n as fp32 rows (3, 4, 6: see glu_act)
+// output column n as fp32 rows; 8: v + bias[n] as fp32 rows (3, 4, 6: see glu_act)
 template <typename T>
 __device__ __forceinline__ void store_out(void* y, long row, long ldy, long n, float v, int epi, DecayGate dg) {
   if (epi == 0) {
     reinterpret_cast<float*>(y)[row * ldy + n] = v;
   } else if (epi == 7) {
     reinterpret_cast<float*>(y)[row * ldy + n] = decay_gate(v, (int)n, dg);
+  } else if (epi == 8) {
+    reinterpret_cast<float*>(y)[row * ldy + n] = v + dg.bias[n];
   } else {
     if (epi == 1) { v = v > 0.f ? v : 0.f; v = v * v; }
     if (epi == 5) v = tanhf(v);
@@ -286,8 +289,8 @@ int launch(const void* x, const void* w, void* y, int M, int N, int K, int epi, 
            int idx_div, int f32, void* stream, int G = 1, long ldx = 0, long gsx = 0, long ldy = 0, long gsy = 0,
            GluClamp gc = GluClamp{nullptr, 0.f, 0.f}, DecayGate dg = DecayGate{nullptr, nullptr, 0}) {
   if (!x || !w || !y) return SSD_ERR_ARG;
-  if (M <= 0 || N <= 0 || K <= 0 || epi < 0 || epi > 7) return SSD_ERR_SHAPE;
-  if (epi == 7 && !dg.rate) return SSD_ERR_SHAPE;
+  if (M <= 0 || N <= 0 || K <= 0 || epi < 0 || epi > 8) return SSD_ERR_SHAPE;
+  if ((epi == 7 && !dg.rate) || (epi == 8 && !dg.bias)) return SSD_ERR_SHAPE;
   if (epi_pairs(epi) && (f32 || (N & 1))) return SSD_ERR_SHAPE;        // the paired epilogues exist in the bf16 forms only
   if (offsets && E <= 0) return SSD_ERR_SHAPE;
   if (G < 1 || G > 65535 || (G > 1 && offsets)) return SSD_ERR_SHAPE;
@@ -368,4 +371,11 @@ extern "C" int ssd_gemm_rows_decay_gate(const void* x_rows, const void* w_rows, 
   if (n_decay < 0 || n_decay > N) return SSD_ERR_SHAPE;
   return launch(x_rows, w_rows, y, M, N, K, 7, nullptr, 0, nullptr, 1, f32, stream, 1, 0, 0, 0, 0, GluClamp{nullptr, 0.f, 0.f},
                 DecayGate{rate, bias, n_decay});
+}
+
+extern "C" int ssd_gemm_rows_bias(const void* x_rows, const void* w_rows, void* y, int M, int N, int K, const float* bias, int f32,
+                                  void* stream) {
+  if (!bias) return SSD_ERR_ARG;
+  return launch(x_rows, w_rows, y, M, N, K, 8, nullptr, 0, nullptr, 1, f32, stream, 1, 0, 0, 0, 0, GluClamp{nullptr, 0.f, 0.f},
+                DecayGate{nullptr, bias, 0});
 }

@@ -1,7 +1,7 @@
 // Kernels of decoders that normalise a sublayer's OUTPUT only and average over the depth:
 //     x <- x + w * rms(f(x))          (the sublayer reads the residual row itself; w = 1 + the stored weight, given as fp32)
 //     after layer i:  X_(i+1) = x,    x <- sum_(j <= i+1) coef[j] * X_j      (X_0 = the embedding output)
-//  * ssd_embed_hist         token rows of the embedding table -> fp32 residual rows, level 0 of the history, GEMM-input rows
+//  * ssd_embed_hist         token rows of the embedding table times a constant -> fp32 residual rows, level 0 of the history, GEMM-input rows
 //  * ssd_postnorm_tail      (routed mix ->) output norm + residual sum (-> history level + depth average) -> the next sublayer's input
 //                           rows (the residual row in the element type), one launch
 //  * ssd_rmsnorm_w32_rows   y = w * x / sqrt(mean(x^2) + eps) with fp32 weights, optional row gather (the model's last norm)
@@ -37,13 +37,13 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 template <typename T>
 __global__ void __launch_bounds__(256)
 embed_hist_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table, float* __restrict__ x, float* __restrict__ hist0,
-                  T* __restrict__ rows, int W, long vocab) {
+                  T* __restrict__ rows, float scale, int W, long vocab) {
   const size_t t = blockIdx.x;
   const long id = ids[t];
   const bool ok = id >= 0 && id < vocab;
   const T* src = table + (size_t)(ok ? id : 0) * W;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < W; c += 256 * gridDim.y) {
-    const float v = ok ? ldf<T>(src + c) : 0.f;
+    const float v = ok ? ldf<T>(src + c) * scale : 0.f;
     x[t * W + c] = v;
     if (hist0) hist0[t * W + c] = v;
     if (rows) stf<T>(rows + t * W + c, v);
@@ -160,17 +160,17 @@ inline int col_blocks(int rows, int cols) { return rows < 64 ? (cols + 255) / 25
 
 #define LAUNCH_OK() (hipGetLastError() == hipSuccess ? SSD_OK : SSD_ERR_LAUNCH)
 
-extern "C" int ssd_embed_hist(const int64_t* ids, const void* table, void* x_out, void* hist0, void* rows_out, int T, int W, long vocab,
-                              int f32, void* stream) {
+extern "C" int ssd_embed_hist(const int64_t* ids, const void* table, void* x_out, void* hist0, void* rows_out, float scale, int T, int W,
+                              long vocab, int f32, void* stream) {
   if (!ids || !table || !x_out) return SSD_ERR_ARG;
   if (T <= 0 || W <= 0 || vocab <= 0) return SSD_ERR_SHAPE;
   const dim3 grid(T, col_blocks(T, W));
   if (f32)
     hipLaunchKernelGGL(embed_hist_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, ids, (const float*)table, (float*)x_out,
-                       (float*)hist0, (float*)rows_out, W, vocab);
+                       (float*)hist0, (float*)rows_out, scale, W, vocab);
   else
     hipLaunchKernelGGL(embed_hist_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, ids, (const bf16_t*)table, (float*)x_out,
-                       (float*)hist0, (bf16_t*)rows_out, W, vocab);
+                       (float*)hist0, (bf16_t*)rows_out, scale, W, vocab);
   return LAUNCH_OK();
 }
 

@@ -11,7 +11,7 @@
 //  state space          ssd_ssd_scan           per head, S [N][Dv]:  S_t = exp(-exp(A_log) dt_t) S_(t-1) + dt_t B_t x_t^T,  y_t = S_t^T C_t + D x_t,
 //                                              dt_t = softplus(dt_raw + dt_bias) (no clamp); B / C shared by the heads of a group; also
 //                                              saves the slot's last taps - 1 convolution inputs
-//  output               ssd_group_gate_norm    RMS norm in `groups` equal parts of the row, a gate (silu, sigmoid, or rows that hold the
+//  output               ssd_group_gate_norm    (each part divided by a per-row number,) RMS norm in `groups` equal parts of the row, a gate (silu, sigmoid, or rows that hold the
 //                                              factor itself) either BEFORE the norm (gate_first) or after it, times a weight (per column,
 //                                              or repeated every w_period columns) and a constant, as GEMM-input rows with a row stride
 // Everything that enters a recurrence is fp32: the projections' fp32 accumulators come in as fp32 rows, decays, step sizes, states and
@@ -323,20 +323,21 @@ __device__ __forceinline__ float gate_act(float z, int act) {
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-group_gate_norm_kernel(const float* __restrict__ o, const float* __restrict__ gate, long ldg, int act, const T* __restrict__ w, int w_period,
+group_gate_norm_kernel(const float* __restrict__ o, const float* __restrict__ den, const float* __restrict__ gate, long ldg, int act, const T* __restrict__ w, int w_period,
                        float eps, float scale, T* __restrict__ out, long ldo, int N, int groups, int gate_first) {
   const size_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, per = N / groups;
   const float* orow = o + t * N;
   const float* grow = gate + t * ldg;
   for (int g = blockIdx.y * 4 + wave; g < groups; g += 4 * gridDim.y) {
+    const float dv = den ? 1.0f / den[t * groups + g] : 1.0f;
     float ss = 0.f;
     for (int c = g * per + lane; c < (g + 1) * per; c += 64) {
-      const float v = gate_first ? orow[c] * gate_act(grow[c], act) : orow[c];
+      const float v = gate_first ? orow[c] * dv * gate_act(grow[c], act) : orow[c] * dv;
       ss += v * v;
     }
     ss = wave_sum(ss);
-    const float r = 1.0f / sqrtf(ss / (float)per + eps);
+    const float r = 1.0f / sqrtf(ss / (float)per + eps) * dv;
     for (int c = g * per + lane; c < (g + 1) * per; c += 64) {
       const float gs = gate_act(grow[c], act), wv = ldf<T>(w + (w_period ? c % w_period : c));
       const float v = gate_first ? orow[c] * gs * r * wv : orow[c] * r * wv * gs;
@@ -469,20 +470,20 @@ extern "C" int ssd_ssd_scan(const void* xbc_rows, long ldx, int x_off, int b_off
   return LAUNCH_OK();
 }
 
-extern "C" int ssd_group_gate_norm(const void* o_rows, const void* gate_rows, long ldg, int gate_act, const void* weight, int w_period,
-                                   float eps, float out_scale, void* out_rows, long ldo, int T, int N, int groups, int gate_first, int f32,
-                                   void* stream) {
+extern "C" int ssd_group_gate_norm(const void* o_rows, const float* den_rows, const void* gate_rows, long ldg, int gate_act,
+                                   const void* weight, int w_period, float eps, float out_scale, void* out_rows, long ldo, int T, int N,
+                                   int groups, int gate_first, int f32, void* stream) {
   if (!o_rows || !gate_rows || !weight || !out_rows) return SSD_ERR_ARG;
   if (T <= 0 || N <= 0 || groups <= 0 || N % groups || ldg < N || ldo < N || gate_act < 0 || gate_act > 2 || w_period < 0)
     return SSD_ERR_SHAPE;
   const int gb = (groups + 3) / 4;
   const dim3 grid(T, T >= 256 ? 1 : (gb < 16 ? gb : 16));
   if (f32)
-    hipLaunchKernelGGL(group_gate_norm_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows,
+    hipLaunchKernelGGL(group_gate_norm_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows, den_rows,
                        (const float*)gate_rows, ldg, gate_act, (const float*)weight, w_period, eps, out_scale, (float*)out_rows, ldo, N,
                        groups, gate_first);
   else
-    hipLaunchKernelGGL(group_gate_norm_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows,
+    hipLaunchKernelGGL(group_gate_norm_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, (const float*)o_rows, den_rows,
                        (const float*)gate_rows, ldg, gate_act, (const bf16_t*)weight, w_period, eps, out_scale, (bf16_t*)out_rows, ldo, N,
                        groups, gate_first);
   return LAUNCH_OK();

@@ -46,6 +46,9 @@ def model_class(family: str):
     if family == "dusupel":
         from ssd_amd.dusupel import HipDusupel
         return HipDusupel
+    if family == "tumudra":
+        from ssd_amd.tumudra import HipTumudra
+        return HipTumudra
     return HipDecoder
 
 

@@ -16,7 +16,7 @@ _LIB = None
 
 c_void_p, c_int, c_long, c_float, c_int64 = C.c_void_p, C.c_int, C.c_long, C.c_float, C.c_int64
 
-ABI_VERSION = 7       # include/ssd_hip.h SSD_HIP_ABI_VERSION (tests/test_abi.py compares the two)
+ABI_VERSION = 8       # include/ssd_hip.h SSD_HIP_ABI_VERSION (tests/test_abi.py compares the two)
 
 # name -> argtypes, exactly include/ssd_hip.h (+ include/ssd_hip_tune.h)
 SIGNATURES = {
@@ -155,7 +155,7 @@ SIGNATURES = {
                           c_int, c_void_p],
     "ssd_winattn_paged": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                           c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_long, c_float, c_void_p,
-                          c_long, c_int, c_void_p],
+                          c_long, c_int, c_void_p, c_long, c_void_p],
     "ssd_winattn_store_conv_rope": [c_void_p, c_long, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                     c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                     c_int, c_void_p],
@@ -163,7 +163,7 @@ SIGNATURES = {
                                c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ssd_moe_route_sigmoid_grouped": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ssd_gemm_rows_glu_clamp": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_void_p],
-    "ssd_embed_hist": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_long, c_int, c_void_p],
+    "ssd_embed_hist": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_long, c_int, c_void_p],
     "ssd_postnorm_tail": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_long, c_int, c_void_p,
                           c_void_p, c_int, c_int, c_int, c_void_p],
     "ssd_rmsnorm_w32_rows": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -177,8 +177,8 @@ SIGNATURES = {
                              c_void_p, c_int, c_int, c_int, c_void_p],
     "ssd_ssd_scan": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                      c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
-    "ssd_group_gate_norm": [c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_float, c_float, c_void_p, c_long, c_int, c_int, c_int,
-                            c_int, c_int, c_void_p],
+    "ssd_group_gate_norm": [c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_float, c_float, c_void_p, c_long, c_int, c_int,
+                            c_int, c_int, c_int, c_void_p],
     "ssd_gemm_rows_decay_gate": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "ssd_delta_prep": [c_void_p, c_long, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                        c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
@@ -190,6 +190,16 @@ SIGNATURES = {
     "ssd_lnorm_tail": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int,
                        c_void_p],
     "ssd_lnorm_rows": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p],
+    "ssd_gemm_rows_bias": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p],
+    "ssd_winattn_store_norm_rope": [c_void_p, c_long, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
+                                    c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "ssd_memory_gates": [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
+                         c_void_p, c_int, c_int, c_int, c_void_p],
+    "ssd_memory_scan": [c_void_p, c_long, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float,
+                        c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                        c_void_p],
+    "ssd_lnorm_post_tail": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_float, c_void_p, c_int, c_int, c_int,
+                            c_void_p],
     "ssd_draft_advance": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int,
                           c_void_p, c_int, c_void_p],
 }
@@ -209,6 +219,7 @@ FAMILY_SOURCES = {
     "dosuvik": _COMMON_ROWS + ["postnorm.hip", "prenorm.hip", "dyt.hip", "attention_window.hip", "attention_latent.hip", "lightning.hip",
                                "recurrent.hip"],
     "dusupel": _COMMON_ROWS + ["layernorm.hip", "dyt.hip", "attention_window.hip", "delta.hip", "recurrent.hip"],
+    "tumudra": _COMMON_ROWS + ["layernorm.hip", "postnorm.hip", "attention_window.hip", "memory_scan.hip", "recurrent.hip"],
 }
 
 

@@ -413,6 +413,11 @@ def gemm_rows(x, w, y, M: int, N: int, K: int, f32: bool, epilogue: int = GR_F32
     _check(load_library().ssd_gemm_rows(_p(x), _p(w), _p(y), M, N, K, epilogue, int(f32), _stream()), "ssd_gemm_rows")
 
 
+def gemm_rows_bias(x, w, y, M: int, N: int, K: int, bias, f32: bool):
+    """y fp32 = x w^T + bias (fp32 [N])."""
+    _check(load_library().ssd_gemm_rows_bias(_p(x), _p(w), _p(y), M, N, K, _p(bias), int(f32), _stream()), "ssd_gemm_rows_bias")
+
+
 def gemm_rows_grouped(x, w, y, offsets, E: int, rows: int, N: int, K: int, f32: bool, epilogue: int = GR_F32, row_idx=None,
                       idx_div: int = 1):
     _check(load_library().ssd_gemm_rows_grouped(_p(x), _p(w), _p(y), _p(offsets), E, _p(row_idx), idx_div, rows, N, K, epilogue,
@@ -575,14 +580,17 @@ def winattn_store(qkv, ld: int, eps: float, slots, q_out, k_cache, v_cache, T: i
 
 def winattn_paged(q, k_cache, v_cache, slopes, sinks, block_tables, max_blocks: int, positions, B: int, T: int, H: int, G: int, D: int,
                   Dv: int, block_size: int, window: int, scale: float, cap: float, out_rows, f32: bool, cu_q=None, q_per_seq: int = 0,
-                  max_q: int = 0, out_freqs=None, keep_first: int = 0, gate=None, ldg: int = 0, out_scale: float = 1.0, ldo: int = 0):
+                  max_q: int = 0, out_freqs=None, keep_first: int = 0, gate=None, ldg: int = 0, out_scale: float = 1.0, ldo: int = 0,
+                  workspace=None):
     """max_q > 0 (an upper bound of the rows a sequence brings; bf16, aligned head sizes, block_size % 32 == 0): the MFMA form.
     out_freqs (fp32 [Dv / 2]): every head's output turns back by the query's position (values cached rotated by their own).
     keep_first: so many first tokens of a sequence stay visible whatever the window.  gate (fp32 rows, stride ldg): outputs times
-    sigmoid(gate) * out_scale.  ldo: row stride of out_rows (0: H * Dv)."""
+    sigmoid(gate) * out_scale.  ldo: row stride of out_rows (0: H * Dv).  workspace (fp32): decode batches may cut a sequence's keys over
+    workgroups."""
     _check(load_library().ssd_winattn_paged(_p(q), _p(k_cache), _p(v_cache), _p(slopes), _p(sinks), _p(block_tables), max_blocks,
                                             _p(positions), _p(cu_q), q_per_seq, max_q, B, T, H, G, D, Dv, block_size, window, keep_first, scale,
-                                            cap, _p(out_freqs), _p(gate), ldg, out_scale, _p(out_rows), ldo or H * Dv, int(f32), _stream()),
+                                            cap, _p(out_freqs), _p(gate), ldg, out_scale, _p(out_rows), ldo or H * Dv, int(f32), _p(workspace),
+                                            workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream()),
            "ssd_winattn_paged")
 
 
@@ -593,6 +601,14 @@ def winattn_store_conv_rope(proj, ld: int, col_off: int, conv_w, taps: int, conv
                                                       _p(positions), _p(cu_q), q_per_seq, B, _p(qk_freqs), rot_dims, _p(slots), _p(q_out),
                                                       _p(k_cache), _p(v_cache), T, H, G, D, Dv, block_size, int(f32), _stream()),
            "ssd_winattn_store_conv_rope")
+
+
+def winattn_store_norm_rope(qkv, ld: int, q_norm_w, k_norm_w, eps: float, positions, qk_freqs, rot_dims: int, slots, q_out, k_cache, v_cache,
+                            T: int, H: int, G: int, D: int, Dv: int, block_size: int, f32: bool):
+    """G = 0: queries only (k_norm_w, k_cache, v_cache None)."""
+    _check(load_library().ssd_winattn_store_norm_rope(_p(qkv), ld, _p(q_norm_w), _p(k_norm_w), eps, _p(positions), _p(qk_freqs), rot_dims,
+                                                      _p(slots), _p(q_out), _p(k_cache), _p(v_cache), T, H, G, D, Dv, block_size, int(f32),
+                                                      _stream()), "ssd_winattn_store_norm_rope")
 
 
 def winattn_store_rope(qkv, ld: int, q_norm_w, k_norm_w, eps: float, positions, qk_freqs, rot_dims: int, v_freqs, slots, q_out, k_cache,
@@ -634,15 +650,16 @@ GATE_SILU, GATE_SIGMOID, GATE_NONE = 0, 1, 2
 
 
 def group_gate_norm(o_rows, gate_rows, ldg: int, weight, eps: float, out_rows, T: int, N: int, groups: int, gate_first: bool, f32: bool,
-                    gate_act: int = GATE_SILU, w_period: int = 0, out_scale: float = 1.0, ldo: int = 0):
-    _check(load_library().ssd_group_gate_norm(_p(o_rows), _p(gate_rows), ldg, gate_act, _p(weight), w_period, eps, out_scale, _p(out_rows),
+                    gate_act: int = GATE_SILU, w_period: int = 0, out_scale: float = 1.0, ldo: int = 0, den=None):
+    """den (fp32 [T][groups]): every part of o is divided by its number first."""
+    _check(load_library().ssd_group_gate_norm(_p(o_rows), _p(den), _p(gate_rows), ldg, gate_act, _p(weight), w_period, eps, out_scale, _p(out_rows),
                                               ldo or N, T, N, groups, int(gate_first), int(f32), _stream()), "ssd_group_gate_norm")
 
 
 # ---- layers that normalise a sublayer's output only, depth-weighted average, retention, grouped sigmoid router ----
 
-def embed_hist(ids, table, x_out, T: int, W: int, f32: bool, hist0=None, rows_out=None):
-    _check(load_library().ssd_embed_hist(_p(ids), _p(table), _p(x_out), _p(hist0), _p(rows_out), T, W, table.shape[0], int(f32), _stream()),
+def embed_hist(ids, table, x_out, T: int, W: int, f32: bool, hist0=None, rows_out=None, scale: float = 1.0):
+    _check(load_library().ssd_embed_hist(_p(ids), _p(table), _p(x_out), _p(hist0), _p(rows_out), scale, T, W, table.shape[0], int(f32), _stream()),
            "ssd_embed_hist")
 
 
@@ -719,3 +736,27 @@ def lnorm_tail(x, y_rows, mult: float, eps: float, T: int, W: int, f32: bool, no
 def lnorm_rows(x, weight, bias, out_rows, eps: float, T: int, W: int, f32: bool, gather=None):
     _check(load_library().ssd_lnorm_rows(_p(x), _p(weight), _p(bias), _p(out_rows), _p(gather), eps, T, W, int(f32), _stream()),
            "ssd_lnorm_rows")
+
+
+def lnorm_post_tail(x, y_rows, weight, eps: float, T: int, W: int, f32: bool, *, y2_rows=None, w1=None, w2=None, pair_scale: float = 1.0,
+                    next_out=None):
+    """x += weight * layer norm of (y_rows | pair_scale * (w1 * rms(y_rows) + w2 * rms(y2_rows))); next_out = x as element-type rows."""
+    _check(load_library().ssd_lnorm_post_tail(_p(x), _p(y_rows), _p(y2_rows), _p(w1), _p(w2), pair_scale, _p(weight), eps, _p(next_out), T, W,
+                                              int(f32), _stream()), "ssd_lnorm_post_tail")
+
+
+# ---- linear attention over an outer-product memory: exponential gates with a normaliser, or a fixed decay per head ----
+
+def memory_gates(proj, ld: int, i_off: int, f_off: int, bias_i, bias_f, cap: float, positions, state_slots, m_state, gates, B: int, H: int,
+                 Dv: int, cu_q=None, q_per_seq: int = 0):
+    _check(load_library().ssd_memory_gates(_p(proj), ld, i_off, f_off, _p(bias_i), _p(bias_f), cap, _p(positions), _p(cu_q), q_per_seq,
+                                           _p(state_slots), _p(m_state), _p(gates), B, H, Dv, _stream()), "ssd_memory_gates")
+
+
+def memory_scan(proj, ld: int, q_off: int, k_off: int, v_off: int, positions, state_slots, state, out_rows, B: int, H: int, D: int, Dv: int,
+                DP: int, *, q_scale: float = 1.0, decay=None, gates=None, i_off: int = 0, f_off: int = 0, bias_i=None, bias_f=None,
+                cap: float = 0.0, m_state=None, den=None, cu_q=None, q_per_seq: int = 0):
+    """decay (fp32 [H]): fixed decays; else exponential gates from the projections at i_off / f_off (or the rows of memory_gates)."""
+    _check(load_library().ssd_memory_scan(_p(proj), ld, q_off, k_off, v_off, q_scale, _p(decay), _p(gates), i_off, f_off, _p(bias_i),
+                                          _p(bias_f), cap, _p(positions), _p(cu_q), q_per_seq, _p(state_slots), _p(state), _p(m_state),
+                                          _p(out_rows), _p(den), B, H, D, Dv, DP, _stream()), "ssd_memory_scan")

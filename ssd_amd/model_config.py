@@ -541,14 +541,34 @@ class FomunexConfig:
 @dataclass
 class Rotary:
     """Rotary positions on the first `dims` entries of a head: pair i turns by position * base^(-2i/dims).  layout "halves" pairs
-    entry i with i + dims / 2, "interleaved" pairs entry 2i with 2i + 1."""
+    entry i with i + dims / 2, "interleaved" pairs entry 2i with 2i + 1.  scaling (optional) = {factor, low, high, original}: frequencies
+    scaled by wavelength, see frequencies()."""
     dims: int
     base: float
     layout: str = "halves"
+    scaling: dict | None = None
 
     def frequencies(self, dims: int | None = None) -> list[float]:
+        """scaling: a pair whose wavelength l = 2 pi / f is shorter than original / high keeps f, one longer than original / low gets
+        f / factor, between the two the frequencies are blended linearly in original / l (the Llama 3.1 rule)."""
+        import math
         d = self.dims if dims is None else dims
-        return [self.base ** (-2.0 * i / d) for i in range(d // 2)]
+        f = [self.base ** (-2.0 * i / d) for i in range(d // 2)]
+        sc = self.scaling
+        if not sc:
+            return f
+        factor, low, high, orig = (float(sc[k]) for k in ("factor", "low", "high", "original"))
+
+        def scaled(fi: float) -> float:
+            length = 2.0 * math.pi / fi
+            if length < orig / high:
+                return fi
+            if length > orig / low:
+                return fi / factor
+            s = (orig / length - low) / (high - low)
+            return (1.0 - s) * fi / factor + s * fi
+
+        return [scaled(fi) for fi in f]
 
     def to_halves(self, width: int) -> list[int]:
         """The order of a `width`-wide rotated part that turns this layout into the "halves" layout (the identity for "halves"): a dot
@@ -710,6 +730,11 @@ class DosuvikConfig:
 # first tokens, and a gated delta rule with a decay per head); every q / k / v channel passes a short causal convolution; a span of
 # layers may run several passes with the same weights
 # --------------------------------------------------------------------------------------------------
+def padded_channels(dim: int) -> int:
+    """Key channels of a head as the recurrent scans with transposed states lay them out (padded with zeros)."""
+    return 32 if dim <= 32 else -(-dim // 64) * 64
+
+
 @dataclass
 class GatedDelta:
     """Gated delta rule over a recurrent fp32 [dim][vdim] state per head: S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q with
@@ -733,8 +758,7 @@ class GatedDelta:
 
     @property
     def padded_dim(self) -> int:
-        """Key channels of a head as the kernels lay them out (padded with zeros)."""
-        return 32 if self.dim <= 32 else -(-self.dim // 64) * 64
+        return padded_channels(self.dim)
 
 
 @dataclass
@@ -873,9 +897,138 @@ class DusupelConfig:
         return out
 
 
+# --------------------------------------------------------------------------------------------------
+# Tumudra: layers that layer-norm a sublayer's OUTPUT only (x <- x + ln(f(x))) over an fp32 residual; mixers are grouped-query attention
+# with biases, per-head q / k norms and rotary positions (a layer may read another layer's keys and values), retention, or two mixers
+# side by side (windowed attention, and an xLSTM matrix memory with exponential gates), each normed before they are averaged; dense
+# relu^2 feed-forwards
+# --------------------------------------------------------------------------------------------------
+@dataclass
+class HeadNormAttention:
+    """Grouped-query attention whose q and k are RMS-normed per head (one weight vector of size dim for all q heads, one for all k heads)
+    before the rotation; ordinary causal softmax over the last `window` tokens (0: all of them); biases on every projection or on none.
+    kv_from: the layer whose cached keys and values this one reads instead of projecting its own (-1: its own)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rope: Rotary
+    window: int = 0
+    bias: bool = False
+    kv_from: int = -1
+    kind: str = "attention"
+
+
+@dataclass
+class MatrixMemory:
+    """Matrix memory of xLSTM (mLSTM): per head a fp32 [dim][vdim] memory and a normaliser, S <- a S + b k v^T, with exponential input and
+    forget gates whose logits are soft-capped by gate_cap, stabilised by a running maximum; each head's read-out divided by its root mean
+    square, times a weight over all heads, times sigmoid(W_g h)."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+    kind: str = "memory"
+
+
+@dataclass
+class NormedPair:
+    """Two mixers that read the same row: half the sum of their outputs, each RMS-normed over the width with a weight of its own."""
+    left: HeadNormAttention
+    right: MatrixMemory
+    kind: str = "parallel"
+
+
+@dataclass
+class Relu2MLP:
+    """Dense feed-forward W_down relu(W_up h)^2."""
+    ff: int
+    kind: str = "dense"
+
+
+@dataclass
+class TumudraLayer:
+    mixer: object               # HeadNormAttention | RetentionMixer | NormedPair
+    mlp: object                 # Relu2MLP | None
+
+
+@dataclass
+class TumudraConfig:
+    """config.json keys: architecture, vocab, width, norm.eps, embedding.scale, layers[{type, mixer{...}, mlp{kind, ff} | null}]; an
+    attention mixer: heads, kv_heads, dim, vdim, scale, rot{base, dims, scaling?}, mask{size}?, kv_from?."""
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: list = field(default_factory=list)
+    embed_scale: float = 1.0
+    family: str = "tumudra"
+    max_position_embeddings: int = 1 << 20
+    tie_word_embeddings: bool = False
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def recurrent(self) -> bool:
+        """True when some layer keeps a per-sequence state that is not a function of cached pages."""
+        return any(l.mixer.kind != "attention" for l in self.layers)
+
+    def to_dict(self) -> dict:
+        return asdict(self)
+
+    @staticmethod
+    def from_json(cfg: dict) -> "TumudraConfig":
+        def rotary(m, layout: str) -> Rotary:
+            r = m.get("rot") or {"dims": 0, "base": 1.0}
+            out = Rotary(int(r["dims"]), float(r["base"]), layout, dict(r["scaling"]) if r.get("scaling") else None)
+            if out.dims % 2 or not 0 <= out.dims <= int(m["dim"]):
+                raise ValueError("Tumudra: rot.dims must be even and at most the head's size")
+            return out
+
+        def attention(m, layout: str, bias: bool) -> HeadNormAttention:
+            src = m.get("kv_from")
+            a = HeadNormAttention(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]),
+                                  float(m["scale"]) if m.get("scale") is not None else int(m["dim"]) ** -0.5, rotary(m, layout),
+                                  int((m.get("mask") or {}).get("size") or 0), bias, -1 if src is None else int(src))
+            if a.heads % a.kv_heads:
+                raise ValueError("Tumudra: heads must be a multiple of kv_heads")
+            return a
+
+        layers = []
+        for i, lc in enumerate(cfg["layers"]):
+            m, kind = lc["mixer"], lc["type"]
+            if kind == "attention":
+                mixer = attention(m, "halves", True)
+                if mixer.kv_from >= 0:
+                    src = layers[mixer.kv_from].mixer if mixer.kv_from < i else None
+                    if src is None or src.kind != "attention" or src.kv_from >= 0 or \
+                            (src.kv_heads, src.dim, src.vdim) != (mixer.kv_heads, mixer.dim, mixer.vdim):
+                        raise ValueError(f"Tumudra: layer {i} cannot use the keys and values of layer {mixer.kv_from}")
+            elif kind == "parallel":
+                r = m["right"]
+                mixer = NormedPair(attention(m["left"], "interleaved", False),
+                                   MatrixMemory(int(r["heads"]), int(r["dim"]), int(r["vdim"]), float(r["gate_cap"])))
+                if mixer.left.kv_from >= 0 or not mixer.right.gate_cap > 0:
+                    raise ValueError("Tumudra: a side-by-side layer has keys and values of its own and a positive gate_cap")
+            elif kind == "retention":
+                mixer = RetentionMixer(int(m["heads"]), int(m["dim"]), int(m["vdim"]), [float(d) for d in m["decay"]], rotary(m, "halves"))
+                if len(mixer.decay) != mixer.heads:
+                    raise ValueError("Tumudra: one decay per head")
+            else:
+                raise ValueError(f"Tumudra: unknown layer type {kind!r}")
+            ml = lc.get("mlp")
+            if ml is not None and ml.get("kind", "dense") != "dense":
+                raise ValueError(f"Tumudra: unknown feed-forward kind {ml['kind']!r}")
+            layers.append(TumudraLayer(mixer, None if ml is None else Relu2MLP(int(ml["ff"]))))
+        scale = (cfg.get("embedding") or {}).get("scale")
+        return TumudraConfig(int(cfg["vocab"]), int(cfg["width"]), float(cfg["norm"]["eps"]), layers, 1.0 if scale is None else float(scale))
+
+
 # config.json "architecture" values that are read by this package's own readers (everything else goes through transformers' AutoConfig)
 ARCHITECTURES = {"Fatulix": FatulixConfig.from_json, "Zerusun": ZerusunConfig.from_json, "Fomunex": FomunexConfig.from_json,
-                 "Dosuvik": DosuvikConfig.from_json, "Dusupel": DusupelConfig.from_json}
+                 "Dosuvik": DosuvikConfig.from_json, "Dusupel": DusupelConfig.from_json, "Tumudra": TumudraConfig.from_json}
 
 
 def read_native_config(model_dir: str):

@@ -202,6 +202,40 @@ def dusupel_param_shapes(cfg) -> list[tuple[str, tuple[int, ...]]]:
     return out + norm("final.norm") + [("head", (cfg.vocab_size, W))]
 
 
+def tumudra_param_shapes(cfg) -> list[tuple[str, tuple[int, ...]]]:
+    """Tensor names and shapes of a Tumudra checkpoint (model_config.TumudraConfig).  '.b' is a projection's bias; a layer that reads
+    another layer's keys and values has no key and value tensors."""
+    W = cfg.hidden_size
+
+    def attention(p, m):
+        proj = lambda n, rows, cols: [(p + n, (rows, cols))] + ([(p + n + ".b", (rows,))] if m.bias else [])
+        out = proj("q", m.heads * m.dim, W) + [(p + "q.norm", (m.dim,))] + proj("o", W, m.heads * m.vdim)
+        if m.kv_from < 0:
+            out += proj("k", m.kv_heads * m.dim, W) + [(p + "k.norm", (m.dim,))] + proj("v", m.kv_heads * m.vdim, W)
+        return out
+
+    def linear(p, m):
+        nk, nv = m.heads * m.dim, m.heads * m.vdim
+        return [(p + "q", (nk, W)), (p + "k", (nk, W)), (p + "v", (nv, W)), (p + "g", (nv, W)), (p + "o", (W, nv))]
+
+    out = [("embed", (cfg.vocab_size, W))]
+    for i, lc in enumerate(cfg.layers):
+        p, m = f"l{i}.", lc.mixer
+        out.append((p + "norm1", (W,)))
+        if m.kind == "attention":
+            out += attention(p + "mix.", m)
+        elif m.kind == "retention":
+            out += linear(p + "mix.", m)
+        else:
+            r, q = m.right, p + "mix.right."
+            out += attention(p + "mix.left.", m.left) + linear(q, r) + [(q + "norm", (r.heads * r.vdim,))]
+            out += [t for n in "if" for t in ((q + n, (r.heads, W)), (q + n + ".b", (r.heads,)))]
+            out += [(p + "mix.left.out", (W,)), (p + "mix.right.out", (W,))]
+        if lc.mlp is not None:
+            out += [(p + "norm2", (W,)), (p + "mlp.up", (lc.mlp.ff, W)), (p + "mlp.down", (W, lc.mlp.ff))]
+    return out + [("final.norm", (W,)), ("head", (cfg.vocab_size, W))]
+
+
 def param_shapes(cfg: ModelConfig) -> list[tuple[str, tuple[int, ...]]]:
     if cfg.family == "eagle3":
         return eagle_param_shapes(cfg)
@@ -215,6 +249,8 @@ def param_shapes(cfg: ModelConfig) -> list[tuple[str, tuple[int, ...]]]:
         return dosuvik_param_shapes(cfg)
     if cfg.family == "dusupel":
         return dusupel_param_shapes(cfg)
+    if cfg.family == "tumudra":
+        return tumudra_param_shapes(cfg)
     h, hd, nh, nkv, I, V = cfg.hidden_size, cfg.head_dim, cfg.num_heads, cfg.num_kv_heads, cfg.intermediate_size, cfg.vocab_size
     out = [("model.embed_tokens.weight", (V, h))]
     for i in range(cfg.num_layers):
@@ -431,7 +467,7 @@ def synthetic_tensor(name: str, shape, seed: int, std: float, gen_device: str, n
         return torch.full(shape, 0.5, dtype=BF16, device=gen_device)
     if name.endswith(".b") and len(shape) == 1:
         return torch.zeros(shape, dtype=BF16, device=gen_device)
-    if "norm" in name or name.endswith("_ln.weight"):
+    if "norm" in name or name.endswith(("_ln.weight", ".left.out", ".right.out")):         # (norms of the two sides of a layer)
         if norm_jitter == 0.0:
             return torch.ones(shape, dtype=BF16, device=gen_device)
         return (1.0 + norm_jitter * torch.randn(shape, generator=g, device=gen_device, dtype=torch.float32)).to(BF16)
