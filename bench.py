@@ -69,11 +69,11 @@ def parse(argv=None):
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=40)
     ap.add_argument("--warmup", type=int, default=5)
-    ap.add_argument("--workload", default="c4", choices=["c4", "c3", "c2", "c5t", "c4e", "tiny", "tiny-async", "tiny-eagle", "fatulix", "zerusun", "fomunex", "dosuvik", "dusupel"])
-    ap.add_argument("--arch-size", default="all", help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel: one of the sizes in ssd_amd/utils/arch_bench.py SIZES, or all")
-    ap.add_argument("--arch-batch", type=int, default=0, help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel: decode batch (0 = 1 and 8)")
-    ap.add_argument("--arch-only", default="both", choices=["both", "fatulix", "llama", "zerusun", "fomunex", "dosuvik", "dusupel"],
-                    help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel: which family of the pair to run")
+    ap.add_argument("--workload", default="c4", choices=["c4", "c3", "c2", "c5t", "c4e", "tiny", "tiny-async", "tiny-eagle", "fatulix", "zerusun", "fomunex", "dosuvik", "dusupel", "tumudra"])
+    ap.add_argument("--arch-size", default="all", help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel | tumudra: one of the sizes in ssd_amd/utils/arch_bench.py SIZES, or all")
+    ap.add_argument("--arch-batch", type=int, default=0, help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel | tumudra: decode batch (0 = 1 and 8)")
+    ap.add_argument("--arch-only", default="both", choices=["both", "fatulix", "llama", "zerusun", "fomunex", "dosuvik", "dusupel", "tumudra"],
+                    help="--workload fatulix | zerusun | fomunex | dosuvik | dusupel | tumudra: which family of the pair to run")
     ap.add_argument("--k", type=int, default=None, help="speculation length (default: 7 async, 6 sync)")
     ap.add_argument("--f", type=int, default=3, help="async fan-out")
     ap.add_argument("--placement", default="auto", choices=["auto", "colocated", "dedicated"])
@@ -448,6 +448,10 @@ def main():
     if args.workload == "dusupel":      # the Dusupel decoder beside an equal-size Fomunex decoder; single GPU
         from ssd_amd.utils.arch_bench import run_dusupel
         print(json.dumps(run_dusupel(args)), flush=True)
+        return
+    if args.workload == "tumudra":      # the Tumudra decoder beside an equal-size Dusupel decoder; single GPU
+        from ssd_amd.utils.arch_bench import run_tumudra
+        print(json.dumps(run_tumudra(args)), flush=True)
         return
     if args.workload == "zerusun":      # the Zerusun decoder beside an equal-size Fatulix decoder; single GPU
         from ssd_amd.utils.arch_bench import run_zerusun

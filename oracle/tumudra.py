@@ -185,3 +185,96 @@ def forward(cfg: dict, w: dict, tokens, residuals: list | None = None, round_inp
         if residuals is not None:
             residuals.append(x.clone())
     return lin(w, "head", rd(layer_norm(x, w["final.norm"], eps)))
+
+
+# ------------------------------------------------------------------------------------------------------------------
+# small configurations and random weights for the tests
+def dense_mlp(ff=24):
+    return {"kind": "dense", "ff": ff}
+
+
+def rotation(dims=8, base=10000.0, scaling=None):
+    return {"base": base, "dims": dims, **({"scaling": scaling} if scaling else {})}
+
+
+def attention_sizes(heads=4, kv_heads=2, dim=8, vdim=8, scale=None, rot=None, size=None, kv_from=None):
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5 if scale is None else scale,
+            "rot": rot or rotation(dim), **({"mask": {"size": size}} if size else {}), **({"kv_from": kv_from} if kv_from is not None else {})}
+
+
+def attention_layer(mlp=None, **sizes):
+    return {"type": "attention", "mixer": attention_sizes(**sizes), "mlp": mlp}
+
+
+def memory_sizes(heads=2, dim=8, vdim=8, gate_cap=6.0):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": gate_cap}
+
+
+def parallel_layer(left=None, right=None, mlp=None):
+    return {"type": "parallel", "mixer": {"left": left or attention_sizes(size=5), "right": right or memory_sizes()}, "mlp": mlp}
+
+
+def retention_layer(heads=2, dim=8, vdim=8, decay=None, rot=None, mlp=None):
+    decay = [1.0 - 2.0 ** -(2 + 2 * h) for h in range(heads)] if decay is None else decay
+    return {"type": "retention", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": decay, "rot": rot or rotation(dim)}, "mlp": mlp}
+
+
+def make_config(layers, vocab=64, width=32, eps=1e-5, scale=4.0):
+    return {"architecture": "Tumudra", "vocab": vocab, "width": width, "norm": {"eps": eps}, "embedding": {"scale": scale}, "layers": layers}
+
+
+def tensor_shapes(cfg: dict) -> list:
+    W = cfg["width"]
+    out = [("embed", (cfg["vocab"], W))]
+
+    def att(p, m, bias):
+        n = {"q": m["heads"] * m["dim"]}
+        if m.get("kv_from") is None:
+            n.update(k=m["kv_heads"] * m["dim"], v=m["kv_heads"] * m["vdim"])
+        mats = [(p + x, (rows, W)) for x, rows in n.items()] + [(p + "o", (W, m["heads"] * m["vdim"]))]
+        return mats + [(p + x + ".norm", (m["dim"],)) for x in n if x != "v"] + ([(x + ".b", (s[0],)) for x, s in mats] if bias else [])
+
+    def lin(p, m):
+        nk, nv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+        return [(p + "q", (nk, W)), (p + "k", (nk, W)), (p + "v", (nv, W)), (p + "g", (nv, W)), (p + "o", (W, nv))]
+
+    for i, lc in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", lc["mixer"]
+        out.append((p + "norm1", (W,)))
+        if lc["type"] == "attention":
+            out += att(p + "mix.", m, True)
+        elif lc["type"] == "retention":
+            out += lin(p + "mix.", m)
+        else:
+            r, H = p + "mix.right.", m["right"]["heads"]
+            out += att(p + "mix.left.", m["left"], False) + lin(r, m["right"]) + [(r + "norm", (H * m["right"]["vdim"],))]
+            out += [(r + "i", (H, W)), (r + "i.b", (H,)), (r + "f", (H, W)), (r + "f.b", (H,)), (p + "mix.left.out", (W,)), (p + "mix.right.out", (W,))]
+        if lc.get("mlp") is not None:
+            out += [(p + "norm2", (W,)), (p + "mlp.up", (lc["mlp"]["ff"], W)), (p + "mlp.down", (W, lc["mlp"]["ff"]))]
+    return out + [("final.norm", (W,)), ("head", (cfg["vocab"], W))]
+
+
+def random_model(cfg: dict, seed: int = 0) -> dict:
+    """bf16 weights: matrices ~ N(0, 1 / fan_in), smaller where they read the residual row (whose entries grow with the embedding scale);
+    q / k norm weights large enough that single keys carry the output; biases away from zero; forget gates from a few tokens to
+    hundreds."""
+    g = torch.Generator().manual_seed(seed)
+    rn = lambda *s: torch.randn(*s, generator=g, dtype=torch.float32)
+    w = {}
+    for name, shape in tensor_shapes(cfg):
+        if name.endswith((".q.norm", ".k.norm")):
+            t = 1.6 + 0.3 * rn(*shape)
+        elif "norm" in name.rsplit(".", 1)[-1] or name.endswith(".out"):
+            t = 1.0 + 0.2 * rn(*shape)
+        elif name.endswith(".f.b"):
+            t = 1.0 + 2.5 * torch.rand(*shape, generator=g)
+        elif name.endswith(".b"):
+            t = 0.5 * rn(*shape)
+        elif name == "embed":
+            t = 0.5 * rn(*shape)
+        elif name.endswith((".right.i", ".right.f")):
+            t = 0.6 * rn(*shape) / math.sqrt(shape[-1])
+        else:
+            t = rn(*shape) / math.sqrt(shape[-1])
+        w[name] = t.to(torch.bfloat16)
+    return w

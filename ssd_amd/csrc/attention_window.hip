@@ -610,20 +610,19 @@ winattn_merge_kernel(const float* __restrict__ part, const float* __restrict__ s
   if (row >= nrows) return;
   const int token = tok0 + row / R, head = g * R + row % R, stride = 16 * (Dv + 2);
   const float* pr = part + ((((size_t)b * G + g) * dtiles + (row >> 4)) * slices * 16 + (row & 15)) * (Dv + 2);
+  // lane s holds slice s's share (at most 64 slices)
   const float sink = sinks ? sinks[head] : -INFINITY;
-  float M = sink;
-  for (int s = lane; s < slices; s += 64) M = fmaxf(M, pr[(size_t)s * stride + Dv]);
-  M = wave_max(M);
-  float L = sinks ? __expf(sink - M) : 0.f;
-  for (int s = 0; s < slices; ++s) {
-    const float l = pr[(size_t)s * stride + Dv + 1];
-    if (l > 0.f) L = fmaf(l, __expf(pr[(size_t)s * stride + Dv] - M), L);
-  }
+  const float ms = lane < slices ? pr[(size_t)lane * stride + Dv] : -INFINITY, ls = lane < slices ? pr[(size_t)lane * stride + Dv + 1] : 0.f;
+  const float M = fmaxf(wave_max(ms), sink);
+  const float fs = ls > 0.f ? __expf(ms - M) : 0.f;
+  const float L = wave_sum(ls * fs) + (sinks ? __expf(sink - M) : 0.f);
+  const float share = fs / L;
   auto column = [&](int d) {
     float o = 0.f;
+#pragma unroll 8
     for (int s = 0; s < slices; ++s)
-      if (pr[(size_t)s * stride + Dv + 1] > 0.f) o = fmaf(pr[(size_t)s * stride + d], __expf(pr[(size_t)s * stride + Dv] - M), o);
-    return o / L;
+      o = fmaf(pr[(size_t)s * stride + d], __int_as_float(__builtin_amdgcn_readlane(__float_as_int(share), s)), o);
+    return o;
   };
   const int hv = Dv >> 1;
   for (int d = lane; d < Dv; d += 64) {

@@ -12,8 +12,10 @@
 // The state is TRANSPOSED, state[slots][H][columns][DP]: a column's key channels contiguous, padded with zeros to DP (32, or a multiple of
 // 64 up to 512).  A column of S depends on the others only through k, q and the gates: P = 8 or 16 lanes own one (DP / P channels each, in
 // registers), 16 or 32 columns per workgroup, and the read-out's sum over the channels is a few DPP adds inside the wave.  Rows are staged
-// through LDS TB at a time, the next batch travels in registers meanwhile; no barrier between tokens.  The arithmetic of a row does not
-// depend on how a prompt is cut nor on the batch: one chain per state element in token order, sums in a fixed order.
+// through LDS TB at a time, the next batch travels in registers meanwhile; tokens are walked in groups of U whose staged values are read one
+// group ahead (a lone wave per SIMD has nothing else to hide the LDS latency behind) and whose read-outs are summed side by side; no
+// barrier between tokens.  The arithmetic of a row does not depend on how a prompt is cut nor on the batch: one chain per state element in
+// token order, sums in a fixed order (a group's missing tokens carry a = 1 and k = 0, which leaves the state as it is).
 #include "common.h"
 
 namespace {
@@ -25,35 +27,53 @@ struct Gating { const float* bias_i; const float* bias_f; float cap; int i_off, 
 
 __device__ __forceinline__ float log_sigmoid_(float y) { return fminf(y, 0.f) - log1pf(expf(-fabsf(y))); }
 
-// Lane t of a wave holds the gate projections of token t (t < n <= N); m is the running maximum before token 0 and becomes the one after
-// token n - 1.  Returns (a, b, exp(-m_t), 0) of the lane's token.
-template <int N>
-__device__ __forceinline__ float4 gate_chain(float zi, float zf, float cap, int n, float& m) {
-  const int lane = threadIdx.x & 63;
-  const float li = cap * tanhf(zi / cap), lf = log_sigmoid_(cap * tanhf(zf / cap));
-  float mine_x = 0.f, mine_m = 0.f;
-  auto link = [&](int t) {
-    const float f = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(lf), t));
-    const float i = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(li), t));
-    const float x = f + m;
-    m = fmaxf(x, i);
-    mine_x = lane == t ? x : mine_x;
-    mine_m = lane == t ? m : mine_m;
-  };
-  if (n == N) {
+// (log forget gate, log input gate) of one token
+__device__ __forceinline__ float2 log_gates(float zi, float zf, float cap) {
+  return float2{log_sigmoid_(cap * tanhf(zf / cap)), cap * tanhf(zi / cap)};
+}
+// (a, b, exp(-m), 0) of a token from the running maxima before and after it
+__device__ __forceinline__ float4 finish_gates(float2 g, float before, float m) {
+  return float4{expf(g.x + before - m), expf(g.y - m), expf(-m), 0.f};
+}
+// The running maxima over n tokens whose log gates lie in LDS, by ONE lane: top[0] = m, the maximum before the first token, top[t + 1] = the one
+// after token t (an addition and a maximum a token; the reads do not depend on the chain).  Returns the last one.
+__device__ __forceinline__ float chain(const float2* pair, float* top, int n, float m) {
+  constexpr int N = 16;                     // tokens whose log gates are read ahead of the chain
+  top[0] = m;
+  int t = 0;
+  if (n >= N) {
+    float2 g[N], next[N];
 #pragma unroll
-    for (int t = 0; t < N; ++t) link(t);
-  } else {
-    for (int t = 0; t < n; ++t) link(t);
+    for (int u = 0; u < N; ++u) g[u] = pair[u];
+    for (; t + N <= n; t += N) {
+      const int ahead = t + 2 * N <= n ? t + N : t;
+#pragma unroll
+      for (int u = 0; u < N; ++u) next[u] = pair[ahead + u];
+#pragma unroll
+      for (int u = 0; u < N; ++u) {
+        m = fmaxf(g[u].x + m, g[u].y);
+        top[t + u + 1] = m;
+      }
+#pragma unroll
+      for (int u = 0; u < N; ++u) g[u] = next[u];
+    }
   }
-  return float4{expf(mine_x - mine_m), expf(li - mine_m), expf(-mine_m), 0.f};
+  for (; t < n; ++t) {
+    m = fmaxf(pair[t].x + m, pair[t].y);
+    top[t + 1] = m;
+  }
+  return m;
 }
 
-__global__ void __launch_bounds__(64)
+// 256 tokens a chunk: every thread prepares and finishes one token, one lane walks the chain.
+__global__ void __launch_bounds__(256)
 memory_gates_kernel(const float* __restrict__ proj, long ld, Gating gt, const int64_t* __restrict__ positions,
                     const int32_t* __restrict__ cu_q, int q_per_seq, const int32_t* __restrict__ state_slots, float* __restrict__ m_state,
                     float4* __restrict__ gates, int H, int copies, int ld_m) {
-  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  constexpr int N = 256;
+  __shared__ float2 pair[N];
+  __shared__ float top[N + 1];              // top[t + 1] = the running maximum after token t of the chunk
+  const int b = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int row0 = cu_q ? cu_q[b] : b * q_per_seq;
   const int row1 = cu_q ? cu_q[b + 1] : (b + 1) * q_per_seq;
   if (row1 <= row0) return;
@@ -62,19 +82,24 @@ memory_gates_kernel(const float* __restrict__ proj, long ld, Gating gt, const in
   const float bi = gt.bias_i[h], bf = gt.bias_f[h];
   float zi = 0.f, zf = 0.f;
   auto fetch = [&](int r) {
-    const int row = r + lane < row1 ? r + lane : row1 - 1;
+    const int row = r + tid < row1 ? r + tid : row1 - 1;
     zi = proj[(size_t)row * ld + gt.i_off + h] + bi;
     zf = proj[(size_t)row * ld + gt.f_off + h] + bf;
   };
   fetch(row0);
-  for (int r = row0; r < row1; r += 64) {
-    const int n = min(row1 - r, 64);
-    const float ci = zi, cf = zf;
-    if (r + 64 < row1) fetch(r + 64);
-    const float4 g = gate_chain<64>(ci, cf, gt.cap, n, m);
-    if (lane < n) gates[(size_t)(r + lane) * H + h] = g;
+  for (int r = row0; r < row1; r += N) {
+    const int n = min(row1 - r, N);
+    const float2 g = log_gates(zi, zf, gt.cap);
+    pair[tid] = g;
+    if (r + N < row1) fetch(r + N);
+    __syncthreads();
+    if (tid == 0) chain(pair, top, n, m);
+    __syncthreads();
+    m = top[n];
+    if (tid < n) gates[(size_t)(r + tid) * H + h] = finish_gates(g, top[tid], top[tid + 1]);
+    __syncthreads();
   }
-  for (int c = lane; c < copies; c += 64) ms[c] = m;
+  for (int c = tid; c < copies; c += N) ms[c] = m;
 }
 
 struct Rows { const float* proj; long ld; int q_off, k_off, v_off; float q_scale; };
@@ -87,9 +112,15 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
                    const int32_t* __restrict__ state_slots, float* __restrict__ state, float* __restrict__ m_state, int ld_m,
                    float* __restrict__ out, float* __restrict__ den, int H, int D, int Dv) {
   constexpr int D4 = P * NJ, DP = 4 * D4, COLS = 256 / P;      // float4 per key vector, padded channels, columns per workgroup
-  constexpr int F = (TB * DP + 255) / 256, FV = (TB * COLS + 255) / 256;
-  __shared__ float4 sk[TB * D4], sq[TB * D4], ss[TB];
-  __shared__ float sv[TB * COLS], so[TB * COLS];
+  constexpr int F = TB * DP / 256, FV = (TB * COLS + 255) / 256;       // staged q / k and v entries per thread
+  constexpr int U = NJ <= 2 ? 4 : (NJ <= 4 ? 2 : 1);           // tokens of a group
+  static_assert(TB * DP % 256 == 0 && TB % (2 * U) == 0 && U <= P, "");
+  __shared__ float4 sk[TB * D4], sq[TB * D4];
+  __shared__ __attribute__((aligned(16))) float2 ss[TB];              // (a, b) of the batch's tokens
+  __shared__ __attribute__((aligned(16))) float sv[COLS * TB];        // [column][token]
+  __shared__ float sz[TB], so[TB * COLS];
+  __shared__ float2 pair[MODE == MODE_INLINE ? TB : 1];
+  __shared__ float top[MODE == MODE_INLINE ? TB + 1 : 1];
   const int b = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * COLS, tid = threadIdx.x;
   const int col = tid / P, p = tid % P, e = c0 + col;
   const int NC = MODE == MODE_DECAY ? Dv : Dv + 1;
@@ -109,23 +140,38 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
 
   float rk[F], rq[F], rv[FV], zi = 0.f, zf = 0.f;
   float4 rg = float4{0.f, 0.f, 0.f, 0.f};
+  const long step_f = 256 % DP == 0 ? (256 / DP) * in.ld : 0;   // from one staged entry of a thread to its next (DP divides 256)
+  const long step_v = (256 / COLS) * in.ld;
+  const float* hq = in.proj + in.q_off + (long)h * D;
+  const float* hv = in.proj + in.v_off + (long)h * Dv;
+  const long k_from_q = (long)in.k_off - in.q_off;
   auto fetch = [&](int r) {
     const int nb = min(row1 - r, TB);
+    const float* base = hq + (size_t)(r + tid / DP) * in.ld + tid % DP;
+    if (256 % DP == 0 && nb == TB && D == DP) {
 #pragma unroll
-    for (int f = 0; f < F; ++f) {
-      const int i = tid + 256 * f, tt = i / DP, d = i % DP;
-      rq[f] = rk[f] = 0.f;
-      if (tt < nb && d < D) {
-        const float* src = in.proj + (size_t)(r + tt) * in.ld + h * D + d;
-        rq[f] = src[in.q_off];
-        rk[f] = src[in.k_off];
+      for (int f = 0; f < F; ++f) {
+        rq[f] = base[f * step_f];
+        rk[f] = base[f * step_f + k_from_q];
+      }
+    } else {
+#pragma unroll
+      for (int f = 0; f < F; ++f) {
+        const int i = tid + 256 * f, tt = i / DP, d = i % DP;
+        rq[f] = rk[f] = 0.f;
+        if (tt < nb && d < D) {
+          const float* src = hq + (size_t)(r + tt) * in.ld + d;
+          rq[f] = *src;
+          rk[f] = src[k_from_q];
+        }
       }
     }
+    const int c = c0 + tid % COLS;
+    const float* vbase = hv + (size_t)(r + tid / COLS) * in.ld + c;
 #pragma unroll
     for (int f = 0; f < FV; ++f) {
-      const int i = tid + 256 * f, tt = i / COLS, c = c0 + i % COLS;
       rv[f] = c == Dv ? 1.f : 0.f;                              // (past the last column: a column of zeros that is never written)
-      if (tt < nb && c < Dv) rv[f] = in.proj[(size_t)(r + tt) * in.ld + in.v_off + h * Dv + c];
+      if (tid / COLS + f * (256 / COLS) < nb && c < Dv) rv[f] = vbase[f * step_v];
     }
     if (tid < nb) {
       if (MODE == MODE_GATES) rg = gates[(size_t)(r + tid) * H + h];
@@ -139,10 +185,48 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
 #pragma unroll
     for (int f = 0; f < FV; ++f) {
       const int i = tid + 256 * f, tt = i / COLS, c = c0 + i % COLS;
-      if (i >= TB * COLS || tt >= nb) continue;
+      if (tt >= nb) continue;             // (nb <= TB: also the threads past the staged entries)
       if (c < Dv) out[((size_t)(r + tt) * H + h) * Dv + c] = so[i];
       else if (MODE != MODE_DECAY && c == Dv) den[(size_t)(r + tt) * H + h] = so[i];
     }
+  };
+  struct Group { float4 k[U][NJ], q[U][NJ]; float2 g[U]; float v[U]; };
+  auto read = [&](Group& x, int t0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        x.k[u][j] = sk[(t0 + u) * D4 + P * j + p];
+        x.q[u][j] = sq[(t0 + u) * D4 + P * j + p];
+      }
+      x.g[u] = ss[t0 + u];
+      x.v[u] = sv[col * TB + t0 + u];
+    }
+  };
+  auto walk = [&](const Group& x, int t0) {
+    float y[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const float a = x.g[u].x, w = MODE == MODE_DECAY ? x.v[u] : x.v[u] * x.g[u].y;
+      float4 o{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        const float4 k = x.k[u][j], q = x.q[u][j];
+        s[j].x = fmaf(a, s[j].x, k.x * w); s[j].y = fmaf(a, s[j].y, k.y * w);
+        s[j].z = fmaf(a, s[j].z, k.z * w); s[j].w = fmaf(a, s[j].w, k.w * w);
+        o.x = fmaf(s[j].x, q.x, o.x); o.y = fmaf(s[j].y, q.y, o.y);
+        o.z = fmaf(s[j].z, q.z, o.z); o.w = fmaf(s[j].w, q.w, o.w);
+      }
+      y[u] = (o.x + o.y) + (o.z + o.w);
+    }
+    float mine = 0.f;                     // lane u of a column finishes token u of the group
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      float z = col_sum<P>(y[u]) * in.q_scale;
+      if (MODE != MODE_DECAY && e == Dv) z = fmaxf(fabsf(z), sz[t0 + u]) + 1e-6f;
+      mine = p == u ? z : mine;
+    }
+    if (p < U) so[(t0 + p) * COLS + col] = mine;
   };
   fetch(row0);
   for (int r = row0; r < row1; r += TB) {
@@ -151,52 +235,44 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
     if (r > row0) put_out(r - TB, TB);
 #pragma unroll
     for (int f = 0; f < F; ++f) {
-      const int i = tid + 256 * f;
-      if (i < TB * DP) {
-        reinterpret_cast<float*>(sq)[i] = rq[f];
-        reinterpret_cast<float*>(sk)[i] = rk[f];
-      }
+      reinterpret_cast<float*>(sq)[tid + 256 * f] = rq[f];
+      reinterpret_cast<float*>(sk)[tid + 256 * f] = rk[f];
     }
 #pragma unroll
     for (int f = 0; f < FV; ++f)
-      if (tid + 256 * f < TB * COLS) sv[tid + 256 * f] = rv[f];
-    if (MODE == MODE_INLINE && tid < 64) rg = gate_chain<TB>(zi, zf, gt.cap, nb, m);
-    if (MODE != MODE_DECAY && tid < nb) ss[tid] = rg;
+      if (tid + 256 * f < TB * COLS) sv[tid % COLS * TB + tid / COLS + f * (256 / COLS)] = rv[f];
+    if (MODE == MODE_INLINE && tid < 64) {
+      const float2 g = log_gates(zi, zf, gt.cap);
+      if (tid < TB) pair[tid] = g;
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_s_waitcnt(0xc07f);               // lgkmcnt(0): this wave's LDS writes have landed
+      if (tid == 0) m = chain(pair, top, nb, m);
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_s_waitcnt(0xc07f);
+      if (tid < nb) rg = finish_gates(g, top[tid], top[tid + 1]);
+    }
+    if (MODE == MODE_DECAY) rg.x = fixed;
+    if (tid < TB) {
+      ss[tid] = tid < nb ? float2{rg.x, rg.y} : float2{1.f, 0.f};
+      sz[tid] = rg.z;
+    }
     __syncthreads();
     if (r + TB < row1) fetch(r + TB);
-    // the staged values of a token are read one token ahead of their use: the LDS latency hides behind the current token's arithmetic
-    float4 k[NJ], q[NJ], sc;
-    float v;
-    auto read = [&](int tt) {
-#pragma unroll
-      for (int j = 0; j < NJ; ++j) {
-        k[j] = sk[tt * D4 + P * j + p];
-        q[j] = sq[tt * D4 + P * j + p];
-      }
-      if (MODE != MODE_DECAY) sc = ss[tt];
-      v = sv[tt * COLS + col];
-    };
-    auto step = [&](int tt) {
-      const float a = MODE == MODE_DECAY ? fixed : sc.x, w = MODE == MODE_DECAY ? v : v * sc.y, floor_ = MODE == MODE_DECAY ? 0.f : sc.z;
-      float4 o{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int j = 0; j < NJ; ++j) {
-        s[j].x = fmaf(a, s[j].x, k[j].x * w); s[j].y = fmaf(a, s[j].y, k[j].y * w);
-        s[j].z = fmaf(a, s[j].z, k[j].z * w); s[j].w = fmaf(a, s[j].w, k[j].w * w);
-        o.x = fmaf(s[j].x, q[j].x, o.x); o.y = fmaf(s[j].y, q[j].y, o.y);
-        o.z = fmaf(s[j].z, q[j].z, o.z); o.w = fmaf(s[j].w, q[j].w, o.w);
-      }
-      read(min(tt + 1, TB - 1));
-      float y = col_sum<P>((o.x + o.y) + (o.z + o.w)) * in.q_scale;
-      if (MODE != MODE_DECAY && e == Dv) y = fmaxf(fabsf(y), floor_) + 1e-6f;
-      if (p == 0) so[tt * COLS + col] = y;
-    };
-    read(0);
+    Group x0, x1;
+    read(x0, 0);
     if (nb == TB) {
-#pragma unroll 4
-      for (int tt = 0; tt < TB; ++tt) step(tt);
+#pragma unroll
+      for (int t = 0; t < TB; t += 2 * U) {
+        read(x1, t + U);
+        walk(x0, t);
+        if (t + 2 * U < TB) read(x0, t + 2 * U);
+        walk(x1, t + U);
+      }
     } else {
-      for (int tt = 0; tt < nb; ++tt) step(tt);
+      for (int t = 0; t < nb; t += U) {
+        if (t > 0) read(x0, t);
+        walk(x0, t);
+      }
     }
   }
   __syncthreads();
@@ -225,7 +301,7 @@ extern "C" int ssd_memory_gates(const void* proj_rows, long ld, int i_off, int f
   if (B <= 0 || H <= 0 || H > 65535 || Dv <= 0 || !(cap > 0.f) || i_off < 0 || f_off < 0 || ld < (long)i_off + H || ld < (long)f_off + H ||
       (!cu_q && q_per_seq <= 0) || (uintptr_t)gates % 16)
     return SSD_ERR_SHAPE;
-  hipLaunchKernelGGL(memory_gates_kernel, dim3(B, H), dim3(64), 0, (hipStream_t)stream, (const float*)proj_rows, ld,
+  hipLaunchKernelGGL(memory_gates_kernel, dim3(B, H), dim3(256), 0, (hipStream_t)stream, (const float*)proj_rows, ld,
                      Gating{bias_i, bias_f, cap, i_off, f_off}, positions, cu_q, q_per_seq, state_slots, (float*)m_state, (float4*)gates, H,
                      Dv + 1, Dv + 1);
   return LAUNCH_OK();

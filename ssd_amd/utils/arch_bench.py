@@ -20,6 +20,10 @@ family, Zerusun (the same latent attention and linear-attention scan kernels, a 
 --workload dusupel: the Dusupel decoder (parallel layers; windowed attention beside a gated delta rule / gated delta rule with a decay
 per channel; dense silu GLU) beside the closest existing family, Fomunex (the same windowed attention over pages, recurrent scans with a
 short convolution over state slots, the same output norm), at equal parameter count with dense feed-forwards.
+
+--workload tumudra: the Tumudra decoder (output-norm layers; windowed attention beside an xLSTM matrix memory / causal attention /
+retention / causal attention over another layer's keys and values; dense relu^2 feed-forwards) beside the closest existing family,
+Dusupel (attention beside a recurrent mixer over state slots, layer norms, dense feed-forwards), at equal parameter count.
 """
 from __future__ import annotations
 
@@ -34,6 +38,7 @@ from ssd_amd.engine.sequence import Sequence
 from ssd_amd.model_config import ConvWindowAttention, DusupelConfig, DusupelLayer, GatedDelta, SideBySide, SiluGluMLP
 from ssd_amd.model_config import (BiasedGroupRoutedMLP, ClampedGluMLP, DosuvikConfig, DosuvikLayer, GatedLatentAttention, RetentionMixer,
                                   Rotary, RotaryWindowAttention)
+from ssd_amd.model_config import HeadNormAttention, MatrixMemory, NormedPair, Relu2MLP, TumudraConfig, TumudraLayer
 from ssd_amd.model_config import (DiffAttention, FatulixConfig, FatulixLayer, FomunexConfig, FomunexLayer, GroupRoutedMLP, LatentAttention,
                                   LightningAttention, Mamba2Mixer, ModelConfig, PolyNormMLP, RopeSpec, RoutedMLP, SigmoidRoutedMLP,
                                   WindowAttention, WkvMixer, ZerusunConfig, ZerusunLayer)
@@ -114,6 +119,24 @@ def dusupel_models(size: str):
     count = lambda cfg: sum(_numel(s) for n, s in param_shapes(cfg) if n not in ("embed", "pos", "head"))
     ff = (count(dus) - count(fom(64))) // (2 * W * L) + 64
     return dus, fom(ff // 64 * 64)
+
+
+def tumudra_models(size: str):
+    """(Tumudra, Dusupel) of equal size: the same width, layers, vocabulary, attention heads, window of the side-by-side layer and state sizes
+    (its recurrent side, and the recurrent layer's); Tumudra's feed-forwards as wide as makes the parameter counts equal."""
+    from ssd_amd.weights import param_shapes
+    W, L, Hh, G, _, _, _, _, _ = SIZES[size]
+    dus, _ = dusupel_models(size)
+    wavelengths = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}
+    att = lambda src: HeadNormAttention(Hh, G, 128, 128, 128 ** -0.5, Rotary(128, 5e5), 0, True, src)
+    par = NormedPair(HeadNormAttention(Hh, G, 128, 128, 128 ** -0.5, Rotary(64, 1e6, "interleaved", wavelengths), 1024),
+                     MatrixMemory(Hh // 2, 128, 128, 15.0))
+    ret = RetentionMixer(Hh, 128, 128, [1.0 - 2.0 ** -(3 + 5 * h / Hh) for h in range(Hh)], Rotary(128, 1e6))
+    mixers = [m for i in range(0, L, 4) for m in (par, att(-1), ret, att(i + 1))][:L]
+    tum = lambda ff: TumudraConfig(VOCAB, W, 1e-5, [TumudraLayer(m, Relu2MLP(ff)) for m in mixers], W ** 0.5)
+    count = lambda cfg: sum(_numel(s) for n, s in param_shapes(cfg) if n not in ("embed", "head"))
+    ff = (count(dus) - count(tum(64))) // (2 * W * L) + 64
+    return tum(ff // 64 * 64), dus
 
 
 def _numel(shape) -> int:
@@ -252,33 +275,43 @@ def run_dosuvik(args) -> dict:
             "closest_model_value": results[k]["zerusun_equal_size"]["decode_tok_s"], "sizes": results}
 
 
-def run_dusupel(args) -> dict:
-    """bench.py --workload dusupel: the Dusupel decoder beside an equal-size Fomunex decoder."""
+def _run_pair(args, name: str, other: str, pair, what: str) -> dict:
+    """A family beside its closest one: pair(size) gives the two configurations, `what` describes the layers in the metric's name."""
     sizes = list(SIZES) if args.arch_size == "all" else [args.arch_size]
     batches = [args.arch_batch] if args.arch_batch else [1, 8]
     only = getattr(args, "arch_only", "both")
     prompt_len, steps, warmup = 2048, max(args.steps, 8), max(args.warmup, 2)
     results = {}
     for size in sizes:
-        dus, fom = dusupel_models(size)
+        mine, closest = pair(size)
         for b in batches:
             key = f"{size}_b{b}"
             results[key] = {}
-            if only in ("both", "dusupel"):
-                results[key]["dusupel"] = measure(dus, prompt_len, b, steps, warmup)
-            if only in ("both", "fomunex"):
-                results[key]["fomunex_equal_size"] = measure(fom, prompt_len, b, steps, warmup)
+            if only in ("both", name):
+                results[key][name] = measure(mine, prompt_len, b, steps, warmup)
+            if only in ("both", other):
+                results[key][f"{other}_equal_size"] = measure(closest, prompt_len, b, steps, warmup)
             print(f"[arch_bench] {key}: {json.dumps(results[key])}", flush=True)
     k = "w4096_b8"
     if k not in results or len(results[k]) < 2:
-        return {"metric": "Dusupel / equal-size Fomunex throughput (partial run)", "sizes": results}
-    return {"metric": "decode tokens/s, Dusupel w4096 (4 layers: attention beside delta rule / channel-decay delta rule, dense GLU), batch 8, "
-                      "beside an equal-size Fomunex decoder",
-            "value": results[k]["dusupel"]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
-            "ms_per_step": results[k]["dusupel"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+        return {"metric": f"{name.capitalize()} / equal-size {other.capitalize()} throughput (partial run)", "sizes": results}
+    return {"metric": f"decode tokens/s, {name.capitalize()} w4096 (4 layers: {what}), batch 8, beside an equal-size {other.capitalize()} decoder",
+            "value": results[k][name]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
+            "ms_per_step": results[k][name]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
             "vs_baseline": None, "dtype": "bf16", "data": "synthetic (random weights, random tokens)",
-            "config": {"model": "dusupel-w4096-synthetic", "global_batch": 8, "seq_len": prompt_len, "parallelism": "single GPU"},
-            "closest_model_value": results[k]["fomunex_equal_size"]["decode_tok_s"], "sizes": results}
+            "config": {"model": f"{name}-w4096-synthetic", "global_batch": 8, "seq_len": prompt_len, "parallelism": "single GPU"},
+            "closest_model_value": results[k][f"{other}_equal_size"]["decode_tok_s"], "sizes": results}
+
+
+def run_dusupel(args) -> dict:
+    """bench.py --workload dusupel: the Dusupel decoder beside an equal-size Fomunex decoder."""
+    return _run_pair(args, "dusupel", "fomunex", dusupel_models, "attention beside delta rule / channel-decay delta rule, dense GLU")
+
+
+def run_tumudra(args) -> dict:
+    """bench.py --workload tumudra: the Tumudra decoder beside an equal-size Dusupel decoder."""
+    return _run_pair(args, "tumudra", "dusupel", tumudra_models, "attention beside matrix memory / attention / retention / attention over shared "
+                     "keys and values, dense relu^2")
 
 
 def run_fomunex(args) -> dict:
