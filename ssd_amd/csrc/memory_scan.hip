@@ -27,9 +27,10 @@ struct Gating { const float* bias_i; const float* bias_f; float cap; int i_off, 
 
 __device__ __forceinline__ float log_sigmoid_(float y) { return fminf(y, 0.f) - log1pf(expf(-fabsf(y))); }
 
-// (log forget gate, log input gate) of one token
-__device__ __forceinline__ float2 log_gates(float zi, float zf, float cap) {
-  return float2{log_sigmoid_(cap * tanhf(zf / cap)), cap * tanhf(zi / cap)};
+// cap * tanh(z / cap): absolute error of a few ulp of cap, which is what an exponent's error counts in
+__device__ __forceinline__ float soft_cap_(float z, float cap) {
+  const float e = expf(-2.0f * fabsf(z) / cap);
+  return copysignf(cap * ((1.0f - e) / (1.0f + e)), z);
 }
 // (a, b, exp(-m), 0) of a token from the running maxima before and after it
 __device__ __forceinline__ float4 finish_gates(float2 g, float before, float m) {
@@ -89,7 +90,7 @@ memory_gates_kernel(const float* __restrict__ proj, long ld, Gating gt, const in
   fetch(row0);
   for (int r = row0; r < row1; r += N) {
     const int n = min(row1 - r, N);
-    const float2 g = log_gates(zi, zf, gt.cap);
+    const float2 g{log_sigmoid_(soft_cap_(zf, gt.cap)), soft_cap_(zi, gt.cap)};
     pair[tid] = g;
     if (r + N < row1) fetch(r + N);
     __syncthreads();
@@ -113,12 +114,12 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
                    float* __restrict__ out, float* __restrict__ den, int H, int D, int Dv) {
   constexpr int D4 = P * NJ, DP = 4 * D4, COLS = 256 / P;      // float4 per key vector, padded channels, columns per workgroup
   constexpr int F = TB * DP / 256, FV = (TB * COLS + 255) / 256;       // staged q / k and v entries per thread
-  constexpr int U = NJ <= 2 ? 4 : (NJ <= 4 ? 2 : 1);           // tokens of a group
-  static_assert(TB * DP % 256 == 0 && TB % (2 * U) == 0 && U <= P, "");
+  constexpr int U = NJ == 1 ? 4 : (NJ == 2 ? 2 : 1);           // tokens of a group
+  static_assert(TB <= 32 && TB * DP % 256 == 0 && TB % (2 * U) == 0 && U <= P, "");
   __shared__ float4 sk[TB * D4], sq[TB * D4];
   __shared__ __attribute__((aligned(16))) float2 ss[TB];              // (a, b) of the batch's tokens
   __shared__ __attribute__((aligned(16))) float sv[COLS * TB];        // [column][token]
-  __shared__ float sz[TB], so[TB * COLS];
+  __shared__ float sz[2][TB], so[TB * COLS];        // exp(-m) (the batches alternate: read while the next batch is staged); read-outs
   __shared__ float2 pair[MODE == MODE_INLINE ? TB : 1];
   __shared__ float top[MODE == MODE_INLINE ? TB + 1 : 1];
   const int b = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * COLS, tid = threadIdx.x;
@@ -136,9 +137,9 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
   float* mp = MODE == MODE_INLINE ? m_state + ((size_t)slot * H + h) * ld_m + blockIdx.z : nullptr;
   float m = MODE == MODE_INLINE && !fresh ? *mp : 0.f;          // every column block keeps a copy: none reads what another one writes
   const float fixed = MODE == MODE_DECAY ? decay[h] : 0.f;
-  const float bi = MODE == MODE_INLINE ? gt.bias_i[h] : 0.f, bf = MODE == MODE_INLINE ? gt.bias_f[h] : 0.f;
+  const float bg = MODE == MODE_INLINE ? (tid < 32 ? gt.bias_f[h] : gt.bias_i[h]) : 0.f;
 
-  float rk[F], rq[F], rv[FV], zi = 0.f, zf = 0.f;
+  float rk[F], rq[F], rv[FV], zg = 0.f;
   float4 rg = float4{0.f, 0.f, 0.f, 0.f};
   const long step_f = 256 % DP == 0 ? (256 / DP) * in.ld : 0;   // from one staged entry of a thread to its next (DP divides 256)
   const long step_v = (256 / COLS) * in.ld;
@@ -175,11 +176,8 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
     }
     if (tid < nb) {
       if (MODE == MODE_GATES) rg = gates[(size_t)(r + tid) * H + h];
-      if (MODE == MODE_INLINE) {
-        zi = in.proj[(size_t)(r + tid) * in.ld + gt.i_off + h] + bi;
-        zf = in.proj[(size_t)(r + tid) * in.ld + gt.f_off + h] + bf;
-      }
     }
+    if (MODE == MODE_INLINE && tid < 64 && tid % 32 < nb) zg = in.proj[(size_t)(r + tid % 32) * in.ld + (tid < 32 ? gt.f_off : gt.i_off) + h] + bg;
   };
   auto put_out = [&](int r, int nb) {
 #pragma unroll
@@ -187,7 +185,7 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
       const int i = tid + 256 * f, tt = i / COLS, c = c0 + i % COLS;
       if (tt >= nb) continue;             // (nb <= TB: also the threads past the staged entries)
       if (c < Dv) out[((size_t)(r + tt) * H + h) * Dv + c] = so[i];
-      else if (MODE != MODE_DECAY && c == Dv) den[(size_t)(r + tt) * H + h] = so[i];
+      else if (MODE != MODE_DECAY && c == Dv) den[(size_t)(r + tt) * H + h] = fmaxf(fabsf(so[i]), sz[(r - row0) / TB & 1][tt]) + 1e-6f;
     }
   };
   struct Group { float4 k[U][NJ], q[U][NJ]; float2 g[U]; float v[U]; };
@@ -222,11 +220,10 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
     float mine = 0.f;                     // lane u of a column finishes token u of the group
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      float z = col_sum<P>(y[u]) * in.q_scale;
-      if (MODE != MODE_DECAY && e == Dv) z = fmaxf(fabsf(z), sz[t0 + u]) + 1e-6f;
+      const float z = col_sum<P>(y[u]);
       mine = p == u ? z : mine;
     }
-    if (p < U) so[(t0 + p) * COLS + col] = mine;
+    if (p < U) so[(t0 + p) * COLS + col] = mine * in.q_scale;
   };
   fetch(row0);
   for (int r = row0; r < row1; r += TB) {
@@ -242,30 +239,31 @@ memory_scan_kernel(Rows in, const float* __restrict__ decay, const float4* __res
     for (int f = 0; f < FV; ++f)
       if (tid + 256 * f < TB * COLS) sv[tid % COLS * TB + tid / COLS + f * (256 / COLS)] = rv[f];
     if (MODE == MODE_INLINE && tid < 64) {
-      const float2 g = log_gates(zi, zf, gt.cap);
-      if (tid < TB) pair[tid] = g;
+      // lanes t and t + 32 prepare token t's forget and input gate
+      const float c = soft_cap_(zg, gt.cap), lf = log_sigmoid_(c);
+      if (tid % 32 < TB) (tid < 32 ? pair[tid % 32].x : pair[tid % 32].y) = tid < 32 ? lf : c;
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_s_waitcnt(0xc07f);               // lgkmcnt(0): this wave's LDS writes have landed
       if (tid == 0) m = chain(pair, top, nb, m);
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_s_waitcnt(0xc07f);
-      if (tid < nb) rg = finish_gates(g, top[tid], top[tid + 1]);
+      if (tid < nb) rg = finish_gates(pair[tid], top[tid], top[tid + 1]);
     }
     if (MODE == MODE_DECAY) rg.x = fixed;
     if (tid < TB) {
       ss[tid] = tid < nb ? float2{rg.x, rg.y} : float2{1.f, 0.f};
-      sz[tid] = rg.z;
+      sz[(r - row0) / TB & 1][tid] = rg.z;
     }
     __syncthreads();
     if (r + TB < row1) fetch(r + TB);
     Group x0, x1;
     read(x0, 0);
     if (nb == TB) {
-#pragma unroll
+#pragma unroll 1
       for (int t = 0; t < TB; t += 2 * U) {
         read(x1, t + U);
         walk(x0, t);
-        if (t + 2 * U < TB) read(x0, t + 2 * U);
+        read(x0, min(t + 2 * U, TB - U));
         walk(x1, t + U);
       }
     } else {
@@ -335,10 +333,20 @@ extern "C" int ssd_memory_scan(const void* proj_rows, long ld, int q_off, int k_
     else if (mode == MODE_GATES) MEMORY(P, NJ, TB, MODE_GATES);         \
     else MEMORY(P, NJ, TB, MODE_INLINE);                                \
   } while (0)
+  if (!cu_q && q_per_seq <= 8 && DP <= 256) {          // decoding: a batch is staged for few tokens
+    switch (DP) {
+      case 32: MEMORY3(8, 1, 8); break;
+      case 64: MEMORY3(16, 1, 8); break;
+      case 128: MEMORY3(16, 2, 8); break;
+      case 192: MEMORY3(16, 3, 8); break;
+      default: MEMORY3(16, 4, 8); break;
+    }
+    return LAUNCH_OK();
+  }
   switch (DP) {
-    case 32: MEMORY3(8, 1, 16); break;
-    case 64: MEMORY3(16, 1, 16); break;
-    case 128: MEMORY3(16, 2, 16); break;
+    case 32: MEMORY3(8, 1, 32); break;
+    case 64: MEMORY3(16, 1, 32); break;
+    case 128: MEMORY3(16, 2, 32); break;
     case 192: MEMORY3(16, 3, 16); break;
     case 256: MEMORY3(16, 4, 16); break;
     case 320: MEMORY3(16, 5, 8); break;

@@ -1000,6 +1000,9 @@ class TumudraConfig:
         for i, lc in enumerate(cfg["layers"]):
             m, kind = lc["mixer"], lc["type"]
             if kind == "attention":
+                if m.get("kv_from") is not None and 0 <= int(m["kv_from"]) < i:      # sizes of keys and values it leaves out: the owner's
+                    owner = cfg["layers"][int(m["kv_from"])]["mixer"]
+                    m = {**{k: owner[k] for k in ("kv_heads", "dim", "vdim", "rot") if k in owner}, **m}
                 mixer = attention(m, "halves", True)
                 if mixer.kv_from >= 0:
                     src = layers[mixer.kv_from].mixer if mixer.kv_from < i else None

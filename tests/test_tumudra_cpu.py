@@ -60,6 +60,10 @@ def test_config_reader_names_and_synthetic_weights(tmp_path):
         breakit(bad)
         with pytest.raises(ValueError):
             TumudraConfig.from_json(bad)
+    short = json.loads(json.dumps(cfg))
+    for k in ("kv_heads", "dim", "vdim", "rot"):                  # what the borrowing layer leaves out equals the owner's
+        del short["layers"][3]["mixer"][k]
+    assert TumudraConfig.from_json(short).layers[3].mixer == a3
     chain = json.loads(json.dumps(cfg))
     chain["layers"].append({**chain["layers"][3], "mixer": {**chain["layers"][3]["mixer"], "kv_from": 3}})
     with pytest.raises(ValueError):               # keys come from a layer that has some

@@ -96,8 +96,8 @@ MEMORY_CASES = [(2, 8, 8), (3, 24, 20), (1, 32, 33), (3, 33, 31), (2, 64, 64), (
 @pytest.mark.parametrize("kind", ["gates", "decay"])
 @pytest.mark.parametrize("Hh,D,Dv", MEMORY_CASES)
 def test_outer_product_memory_in_portions_over_slots(Hh, D, Dv, kind):
-    """Two sequences in slots 2 and 0 of a pool that holds NaN; the first arrives in portions of 1, 2, 37 and 300 rows (one of them beside the
-    second one's rows, one of several staged batches and gate chunks).  Read-out and denominator equal the whole-sequence statement; the rows
+    """Two sequences in slots 2 and 0 of a pool that holds NaN; the first arrives in portions of 1, 2, 37, 8 and 292 rows (one of them beside the
+    second one's rows, one of several staged batches and gate chunks, two in the decoding form).  Read-out and denominator equal the whole-sequence statement; the rows
     of the portions equal those of one whole portion bit by bit; gates computed ahead of the scan equal those inside it bit by bit."""
     gates_on = kind == "gates"
     DP = 32 if D <= 32 else -(-D // 64) * 64
@@ -129,17 +129,18 @@ def test_outer_product_memory_in_portions_over_slots(Hh, D, Dv, kind):
         cu = i32([0] + torch.tensor([x.shape[0] for x, _ in parts]).cumsum(0).tolist())
         T = p.shape[0]
         out, den = (torch.full(s, float("nan"), device=DEV) for s in ((T, Hh * Dv), (T, Hh)))
-        common = dict(i_off=i0, f_off=f0, bias_i=d(bi), bias_f=d(bf), cap=cap, m_state=running, cu_q=d(cu))
+        rows = dict(q_per_seq=T) if len(parts) == 1 and T <= 8 else dict(cu_q=d(cu))         # a fixed row count: the decoding form
+        common = dict(i_off=i0, f_off=f0, bias_i=d(bi), bias_f=d(bf), cap=cap, m_state=running, **rows)
         g = None
         if gates_on and ahead:
             g = torch.full((T, Hh, 4), float("nan"), device=DEV)
             H().memory_gates(d(p), NP, positions=d(pos), state_slots=d(i32(slots)), gates=g, B=len(parts), H=Hh, Dv=Dv, **common)
-        kw = dict(common, gates=g, den=den) if gates_on else dict(decay=d(decay), cu_q=d(cu))
+        kw = dict(common, gates=g, den=den) if gates_on else dict(decay=d(decay), **rows)
         H().memory_scan(d(p), NP, q0, k0, v0, d(pos), d(i32(slots)), state, out, len(parts), Hh, D, Dv, DP, q_scale=qs, **kw)
         return (out.view(T, Hh, Dv) / den.unsqueeze(-1) if gates_on else out.view(T, Hh, Dv)).cpu()
 
     outs, rest, at = [], None, 0
-    for j, n in enumerate((1, 2, 37, 300)):
+    for j, n in enumerate((1, 2, 37, 8, 292)):
         parts, slots = [(pA[at:at + n], at)], [2]
         if j == 1:
             parts.append((pB, 0))
