@@ -71,8 +71,8 @@ def configs():
         # sizes the MFMA attention takes (value tiles that fill and that do not fill the register array; more query heads per key head than a
         # tile has rows), a stacked output product, state rows of 32, 64 and 128 channels
         "fast_forms": F.make_config([P(S(heads=8, kv_heads=2, dim=32, vdim=64, size=70, rot=rot(16)), M(heads=16, dim=32, vdim=32), N(48)),
-                                     A(N(64), heads=4, kv_heads=1, dim=64, vdim=32, rot=rot(64)), R(heads=2, dim=64, vdim=64, rot=rot(32)),
-                                     A(N(32), heads=20, kv_heads=1, dim=64, vdim=32, rot=rot(64), kv_from=1),
+                                     A(N(64), heads=4, kv_heads=1, dim=64, vdim=48, rot=rot(48)), R(heads=2, dim=64, vdim=64, rot=rot(32)),
+                                     A(N(32), heads=20, kv_heads=1, dim=64, vdim=48, rot=rot(48), kv_from=1),
                                      P(S(heads=4, kv_heads=4, dim=96, vdim=96, size=33, rot=rot(96, 1e4, slow)), M(heads=2, dim=128, vdim=32))], vocab=120, width=96),
         "only_attention": F.make_config([A(N(), heads=4, kv_heads=2), A(None, heads=2, kv_heads=2, kv_from=0), A(N(), heads=2, kv_heads=1, dim=16)], vocab=40, width=48),
         "only_recurrent": F.make_config([R(heads=2, dim=12, vdim=20, mlp=N()), R(heads=3, dim=8, vdim=8)], vocab=40, width=48),
